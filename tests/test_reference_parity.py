@@ -11,7 +11,7 @@ import pytest
 
 REF = "/root/reference"
 
-pytestmark = pytest.mark.skipif(not os.path.isdir(REF),
+pytestmark = pytest.mark.skipif(not os.path.isdir(os.path.join(REF, "fei")),
                                 reason="reference tree not mounted")
 
 
