@@ -1,5 +1,10 @@
 """Model specs for the local engine.
 
+Two families of decoder: ``ModelSpec`` (one attention layer repeated;
+Llama-3) and ``TobaraxSpec`` (a list of unlike layers, each with its own
+mixer and sizes, part of the list run several times in a row). ``get_spec``
+takes a registered name or a folder with a config.json.
+
 Llama-3 8B/70B shapes per the BASELINE.json configs (weights are random-init
 — there is no network for checkpoints; bench.py states data=synthetic).
 ``llama3-tiny`` exists for CPU tests; ``bge-base`` shapes the memdir
@@ -8,8 +13,11 @@ embedding encoder (fei_amd/models/bge.py).
 
 from __future__ import annotations
 
-from dataclasses import dataclass
-from typing import Dict
+import json
+import os
+import struct
+from dataclasses import dataclass, fields
+from typing import Any, Dict, List, Optional, Tuple, Union
 
 
 @dataclass(frozen=True)
@@ -46,7 +54,265 @@ class ModelSpec:
         return total * dtype_bytes
 
 
-MODEL_SPECS: Dict[str, ModelSpec] = {
+# -- decoders made of unlike layers -------------------------------------------
+
+@dataclass(frozen=True)
+class LatentAttentionSpec:
+    """Attention whose keys and values are linear maps of a cached latent.
+
+    Per head ``dim`` unrotated and ``rot_dim`` rotated query/key dimensions
+    and ``vdim`` value dimensions; the rotated key part is shared by the
+    heads. ``window``: a query sees that many positions, itself included
+    (None = all)."""
+    heads: int
+    dim: int
+    rot_dim: int
+    vdim: int
+    kv_rank: int
+    scale: float
+    rot_base: float
+    window: Optional[int] = None
+
+    kind = "latent_attention"
+
+    @property
+    def in_rows(self) -> int:
+        """Output rows of the stacked projections of the mixer's input."""
+        return (self.heads * (self.dim + self.rot_dim) + self.kv_rank +
+                self.rot_dim + self.heads * self.vdim)
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def row_width(self) -> int:
+        """Cached values per token."""
+        return self.kv_rank + self.rot_dim
+
+
+@dataclass(frozen=True)
+class GLASpec:
+    """Gated linear attention: a [dim, vdim] state per head, decayed per key
+    channel by sigmoid(z)^(1/tau), z a rank-``gate_rank`` map of the input."""
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
+    gate_rank: int
+
+    kind = "gla"
+
+    @property
+    def in_rows(self) -> int:
+        return (2 * self.heads * self.dim + 2 * self.heads * self.vdim +
+                self.gate_rank)
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def state_size(self) -> int:
+        """State values per sequence."""
+        return self.heads * self.dim * self.vdim
+
+
+MixerSpec = Union[LatentAttentionSpec, GLASpec]
+
+
+@dataclass(frozen=True)
+class LayerSpec:
+    mixer: MixerSpec
+    ff: Optional[int] = None          # width of the feed-forward; None = none
+
+
+@dataclass(frozen=True)
+class LoopSpec:
+    """Layers start .. stop-1 run ``times`` times with the same weights."""
+    start: int
+    stop: int
+    times: int
+
+
+@dataclass(frozen=True)
+class LayerRun:
+    layer: int                        # index into the weights
+    enters_pass: Optional[int] = None  # number of the pass that starts here
+
+
+def _only(d: Dict[str, Any], allowed, where: str) -> None:
+    extra = sorted(set(d) - set(allowed))
+    if extra:
+        raise ValueError(f"unknown keys {extra} in {where}")
+
+
+@dataclass(frozen=True)
+class TobaraxSpec:
+    name: str
+    vocab_size: int
+    hidden_size: int
+    layers: Tuple[LayerSpec, ...]
+    norm_eps: float
+    logit_scale: float
+    logit_softcap: Optional[float] = None
+    loop: Optional[LoopSpec] = None
+    max_seq_len: int = 8192
+    arch: str = "tobarax"
+
+    def __post_init__(self) -> None:
+        if self.loop is not None:
+            lp = self.loop
+            if not (0 <= lp.start < lp.stop <= len(self.layers)
+                    and lp.times >= 1):
+                raise ValueError(f"loop {lp} does not fit "
+                                 f"{len(self.layers)} layers")
+        for L in self.layers:
+            if L.mixer.kind == "latent_attention" and L.mixer.rot_dim % 2:
+                raise ValueError("rotated dimensions come in pairs")
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def intermediate_size(self) -> int:
+        """Widest feed-forward."""
+        return max((L.ff or 0 for L in self.layers), default=0)
+
+    @property
+    def runs(self) -> Tuple[LayerRun, ...]:
+        """Layer runs in execution order; each has its own cache or state."""
+        n, lp = len(self.layers), self.loop
+        if lp is None:
+            return tuple(LayerRun(i) for i in range(n))
+        out: List[LayerRun] = [LayerRun(i) for i in range(lp.start)]
+        for t in range(lp.times):
+            out += [LayerRun(i, t if i == lp.start else None)
+                    for i in range(lp.start, lp.stop)]
+        return tuple(out + [LayerRun(i) for i in range(lp.stop, n)])
+
+    def params_bytes(self, dtype_bytes: int = 2) -> int:
+        C = self.hidden_size
+        total = 2 * self.vocab_size * C + C
+        for L in self.layers:
+            m = L.mixer
+            total += C * m.in_rows + C * m.out_cols + C
+            if m.kind == "latent_attention":
+                total += m.kv_rank * (1 + m.heads * (m.dim + m.vdim))
+            else:
+                total += m.vdim + m.heads * m.dim * (m.gate_rank + 1)
+            if L.ff:
+                total += 3 * C * L.ff + C
+        if self.loop is not None:
+            total += 2 * C * C + self.loop.times * C
+        return total * dtype_bytes
+
+    # -- config.json -----------------------------------------------------------
+
+    @classmethod
+    def from_config(cls, cfg: Dict[str, Any], shapes: Dict[str, Tuple[int, ...]],
+                    name: str = "tobarax",
+                    max_seq_len: int = 8192) -> "TobaraxSpec":
+        """``shapes`` gives the sizes that only the tensors have (the rank of
+        a decay gate). Keys that this class does not know are refused rather
+        than skipped."""
+        _only(cfg, ("architecture", "layers", "logit_scale", "logit_softcap",
+                    "loop", "norm", "vocab", "width", "max_seq_len"), "config")
+        layers = []
+        for i, L in enumerate(cfg["layers"]):
+            where = f"layer {i}"
+            _only(L, ("type", "mixer", "mlp"), where)
+            m, mlp = L["mixer"], L.get("mlp")
+            if L["type"] == "latent_attention":
+                _only(m, ("heads", "dim", "rot_dim", "vdim", "kv_rank",
+                          "scale", "rot", "mask"), where)
+                rot, mask = m.get("rot") or {}, m.get("mask") or {}
+                _only(rot, ("base", "dims"), where)
+                _only(mask, ("size",), where)
+                if rot.get("dims", m["rot_dim"]) != m["rot_dim"]:
+                    raise ValueError(f"{where}: the whole rotated part is "
+                                     "rotated, rot.dims must be rot_dim")
+                mixer: MixerSpec = LatentAttentionSpec(
+                    heads=m["heads"], dim=m["dim"], rot_dim=m["rot_dim"],
+                    vdim=m["vdim"], kv_rank=m["kv_rank"],
+                    scale=float(m["scale"]),
+                    rot_base=float(rot.get("base", 10000.0)),
+                    window=mask.get("size"))
+            elif L["type"] == "gla":
+                _only(m, ("heads", "dim", "vdim", "tau"), where)
+                mixer = GLASpec(
+                    heads=m["heads"], dim=m["dim"], vdim=m["vdim"],
+                    tau=float(m["tau"]),
+                    gate_rank=int(shapes[f"l{i}.mix.a1"][0]))
+            else:
+                raise ValueError(f"{where}: unknown type {L['type']!r}")
+            ff = None
+            if mlp is not None:
+                _only(mlp, ("kind", "ff"), where)
+                if mlp.get("kind", "dense") != "dense":
+                    raise ValueError(f"{where}: unknown mlp {mlp['kind']!r}")
+                ff = int(mlp["ff"])
+            layers.append(LayerSpec(mixer, ff))
+        loop = cfg.get("loop")
+        return cls(
+            name=name, vocab_size=cfg["vocab"], hidden_size=cfg["width"],
+            layers=tuple(layers), norm_eps=float(cfg["norm"]["eps"]),
+            logit_scale=float(cfg.get("logit_scale", 1.0)),
+            logit_softcap=cfg.get("logit_softcap"),
+            loop=LoopSpec(**loop) if loop else None,
+            max_seq_len=int(cfg.get("max_seq_len", max_seq_len)))
+
+    def to_config(self) -> Dict[str, Any]:
+        layers = []
+        for L in self.layers:
+            m = L.mixer
+            if m.kind == "latent_attention":
+                mixer = {"heads": m.heads, "dim": m.dim, "rot_dim": m.rot_dim,
+                         "vdim": m.vdim, "kv_rank": m.kv_rank,
+                         "scale": m.scale,
+                         "rot": {"base": m.rot_base, "dims": m.rot_dim}}
+                if m.window is not None:
+                    mixer["mask"] = {"size": m.window}
+            else:
+                mixer = {"heads": m.heads, "dim": m.dim, "vdim": m.vdim,
+                         "tau": m.tau}
+            layers.append({"type": m.kind, "mixer": mixer,
+                           "mlp": None if L.ff is None else
+                           {"kind": "dense", "ff": L.ff}})
+        out = {"architecture": "Tobarax", "layers": layers,
+               "logit_scale": self.logit_scale,
+               "logit_softcap": self.logit_softcap,
+               "norm": {"eps": self.norm_eps}, "vocab": self.vocab_size,
+               "width": self.hidden_size, "max_seq_len": self.max_seq_len}
+        if self.loop is not None:
+            out["loop"] = {"start": self.loop.start, "stop": self.loop.stop,
+                           "times": self.loop.times}
+        return out
+
+
+AnySpec = Union[ModelSpec, TobaraxSpec]
+
+
+def _tobarax(name: str, vocab: int, width: int, ff: int, heads: int,
+             pattern: str, loop: Optional[LoopSpec], dim: int, rot: int,
+             vdim: int, kv_rank: int, window: int, gla_heads: int,
+             gla_dim: int, gla_vdim: int, gate_rank: int = 16,
+             max_seq_len: int = 8192) -> TobaraxSpec:
+    """``pattern``: one letter per layer, 'a' latent attention, 'g' GLA."""
+    att = LatentAttentionSpec(heads=heads, dim=dim, rot_dim=rot, vdim=vdim,
+                              kv_rank=kv_rank, scale=(dim + rot) ** -0.5,
+                              rot_base=500000.0, window=window)
+    gla = GLASpec(heads=gla_heads, dim=gla_dim, vdim=gla_vdim, tau=16.0,
+                  gate_rank=gate_rank)
+    return TobaraxSpec(
+        name=name, vocab_size=vocab, hidden_size=width,
+        layers=tuple(LayerSpec(att if c == "a" else gla, ff) for c in pattern),
+        norm_eps=1e-5, logit_scale=0.5, logit_softcap=30.0, loop=loop,
+        max_seq_len=max_seq_len)
+
+
+MODEL_SPECS: Dict[str, AnySpec] = {
     "llama3-8b": ModelSpec(
         name="llama3-8b", vocab_size=128256, hidden_size=4096, num_layers=32,
         num_heads=32, num_kv_heads=8, head_dim=128, intermediate_size=14336,
@@ -79,10 +345,61 @@ MODEL_SPECS: Dict[str, ModelSpec] = {
         num_heads=12, num_kv_heads=12, head_dim=64, intermediate_size=3072,
         max_seq_len=512, arch="bert",
     ),
+    # Tobarax: latent-attention and GLA layers, a looped block. The 1b/8b
+    # shapes have the width, feed-forward and vocabulary of the llama3 specs
+    # beside them; tiny is for CPU and numerics tests.
+    "tobarax-tiny": _tobarax(
+        "tobarax-tiny", vocab=320, width=96, ff=160, heads=3, pattern="agga",
+        loop=LoopSpec(1, 3, 2), dim=24, rot=8, vdim=40, kv_rank=56,
+        window=48, gla_heads=2, gla_dim=24, gla_vdim=40, gate_rank=8,
+        max_seq_len=512),
+    "tobarax-1b": _tobarax(
+        "tobarax-1b", vocab=128256, width=2048, ff=8192, heads=16,
+        pattern="ag" * 7, loop=LoopSpec(6, 8, 2), dim=128, rot=64, vdim=128,
+        kv_rank=512, window=1024, gla_heads=8, gla_dim=128, gla_vdim=256),
+    "tobarax-8b": _tobarax(
+        "tobarax-8b", vocab=128256, width=4096, ff=14336, heads=32,
+        pattern="ag" * 15, loop=LoopSpec(14, 16, 2), dim=128, rot=64,
+        vdim=128, kv_rank=512, window=4096, gla_heads=16, gla_dim=128,
+        gla_vdim=256),
 }
 
 
-def get_spec(name: str) -> ModelSpec:
-    if name not in MODEL_SPECS:
-        raise KeyError(f"unknown model {name!r}; known: {sorted(MODEL_SPECS)}")
-    return MODEL_SPECS[name]
+def tensor_shapes(path: str) -> Dict[str, Tuple[int, ...]]:
+    """Names and shapes in a safetensors file, from its header alone."""
+    with open(path, "rb") as f:
+        n = struct.unpack("<Q", f.read(8))[0]
+        if n > 1 << 28:
+            raise ValueError(f"{path}: header of {n} bytes")
+        header = json.loads(f.read(n))
+    return {k: tuple(v["shape"]) for k, v in header.items()
+            if k != "__metadata__"}
+
+
+def load_spec(path: str) -> AnySpec:
+    """Spec of a model folder (config.json + model.safetensors)."""
+    with open(os.path.join(path, "config.json"), encoding="utf-8") as f:
+        cfg = json.load(f)
+    if "arch" in cfg:                      # written by LlamaModel.save_weights
+        known = {f.name for f in fields(ModelSpec)}
+        return ModelSpec(**{k: v for k, v in cfg.items() if k in known})
+    if cfg.get("architecture") == "Tobarax":
+        shapes = tensor_shapes(os.path.join(path, "model.safetensors"))
+        return TobaraxSpec.from_config(
+            cfg, shapes, name=os.path.basename(os.path.abspath(path)))
+    raise ValueError(f"{path}: unknown architecture "
+                     f"{cfg.get('architecture')!r}")
+
+
+def is_model_folder(name: str) -> bool:
+    return os.path.isfile(os.path.join(name, "config.json"))
+
+
+def get_spec(name: str) -> AnySpec:
+    """Spec of a registered model, or of a folder with a config.json."""
+    if name in MODEL_SPECS:
+        return MODEL_SPECS[name]
+    if is_model_folder(name):
+        return load_spec(name)
+    raise KeyError(f"unknown model {name!r}; known: {sorted(MODEL_SPECS)}, "
+                   "or a folder with a config.json")

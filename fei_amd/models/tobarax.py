@@ -1,0 +1,248 @@
+"""Tobarax: a decoder of latent-attention and gated-linear-attention layers.
+
+Each layer adds, to a float32 residual, the outputs of its mixer and of its
+feed-forward, both computed from norms of the same input (so one kernel makes
+both norms, one stacked product makes all projections of the layer, and one
+product over the concatenated outputs adds to the residual). Part of the
+layer list runs several times with the same weights; a pass begins with a
+linear map of the residual and the embedding, and adds a vector of its own.
+
+``forward`` runs one RaggedBatch (engine/step.py): prompts, portions of them
+and decoding sequences, in any mixture. With single tokens only, nothing in it
+depends on host values, so the step can be captured into a hipGraph.
+"""
+
+from __future__ import annotations
+
+import json
+import math
+import os
+from dataclasses import dataclass
+from typing import Callable, Dict, List, Optional
+
+import torch
+
+from fei_amd import ops
+from fei_amd.engine.config import TobaraxSpec
+from fei_amd.engine.kv_cache import HybridCache
+from fei_amd.models.mixers import MIXERS, Mixer
+from fei_amd.ops import reference as ref
+from fei_amd.parallel.pg import ParallelContext
+
+
+@dataclass
+class TobaraxLayer:
+    norm1: torch.Tensor                 # [C] float32
+    norm2: Optional[torch.Tensor]       # [C] float32; None without ff
+    w_in: torch.Tensor                  # [mixer rows + 2 ff, C]
+    w_out: torch.Tensor                 # [C, mixer cols + ff]
+    mixer: Mixer
+
+
+class TobaraxModel:
+    step_cache = True                   # runs RaggedBatches over a HybridCache
+
+    def __init__(self, spec: TobaraxSpec, device: torch.device,
+                 dtype: torch.dtype = torch.bfloat16,
+                 tp: Optional[ParallelContext] = None, seed: int = 1234,
+                 max_seq_len: Optional[int] = None,
+                 weights: Optional[str] = None):
+        if tp is not None and tp.is_distributed:
+            raise ValueError(f"{spec.name}: tensor parallelism is not "
+                             "available for this architecture")
+        self.spec = spec
+        self.device = torch.device(device)
+        self.dtype = dtype
+        self.tp = tp or ParallelContext()
+        self.tp_size = 1
+        # a decay carries every earlier token: the state cannot go back
+        self.recurrent = any(L.mixer.kind == "gla" for L in spec.layers)
+        self._set_weights(self._read(weights) if weights
+                          else self._random(seed))
+        self.resize(max_seq_len or spec.max_seq_len)
+
+    def resize(self, max_seq_len: int) -> None:
+        """Positions up to ``max_seq_len`` - 1 can be run from now on."""
+        self.max_seq_len = max_seq_len
+        keys = {(L.mixer.rot_dim, L.mixer.rot_base) for L in self.spec.layers
+                if L.mixer.kind == "latent_attention"}
+        self._rot = {k: ref.rope_table_exact(max_seq_len, *k,
+                                             device=self.device)
+                     for k in keys}
+
+    # -- weights -------------------------------------------------------------
+
+    def _shapes(self) -> Dict[str, tuple]:
+        s, C = self.spec, self.spec.hidden_size
+        out = {"embed": (s.vocab_size, C), "final.norm": (C,),
+               "head": (s.vocab_size, C)}
+        if s.loop is not None:
+            out["loop.in"] = (C, 2 * C)
+            out["loop.step"] = (s.loop.times, C)
+        for i, L in enumerate(s.layers):
+            out[f"l{i}.norm1"] = (C,)
+            for name, shape in MIXERS[L.mixer.kind].shapes(L.mixer, C).items():
+                out[f"l{i}.mix.{name}"] = shape
+            if L.ff is not None:
+                out[f"l{i}.norm2"] = (C,)
+                out[f"l{i}.mlp.gate"] = (L.ff, C)
+                out[f"l{i}.mlp.up"] = (L.ff, C)
+                out[f"l{i}.mlp.down"] = (C, L.ff)
+        return out
+
+    def _random(self, seed: int) -> Callable[[str], torch.Tensor]:
+        shapes = self._shapes()
+        gen = torch.Generator(device=self.device)
+        gen.manual_seed(seed)
+        depth = math.sqrt(2 * len(self.spec.runs))
+
+        def get(name: str) -> torch.Tensor:
+            shape = shapes[name]
+            if name.endswith(("norm", "norm1", "norm2")):
+                return torch.ones(shape, device=self.device)
+            t = torch.randn(*shape, generator=gen, device=self.device)
+            if name.endswith("a2.b"):
+                return 2.0 + t                   # decays spread below 1
+            if name == "embed":
+                return t
+            scale = 1.0 / math.sqrt(shape[-1])
+            if name.endswith((".o", ".down")):
+                scale /= depth
+            return t * scale
+        return get
+
+    def _read(self, path: str) -> Callable[[str], torch.Tensor]:
+        """Tensors of a model folder, one at a time; names and shapes have to
+        be exactly those of the spec."""
+        from safetensors import safe_open
+
+        f = safe_open(os.path.join(path, "model.safetensors"), framework="pt")
+        shapes = self._shapes()
+        names = set(f.keys())
+        if names != set(shapes):
+            raise ValueError(
+                f"{path}: missing tensors {sorted(set(shapes) - names)[:4]}, "
+                f"unknown tensors {sorted(names - set(shapes))[:4]}")
+
+        def get(name: str) -> torch.Tensor:
+            t = f.get_tensor(name)
+            if tuple(t.shape) != tuple(shapes[name]):
+                raise ValueError(f"{path}: {name} has shape {tuple(t.shape)},"
+                                 f" expected {tuple(shapes[name])}")
+            return t.to(self.device)
+        return get
+
+    def _set_weights(self, get: Callable[[str], torch.Tensor]) -> None:
+        s, dt = self.spec, self.dtype
+        mat = lambda name: get(name).to(dt).contiguous()
+        vec = lambda name: get(name).float().contiguous()
+        self.emb = mat("embed")
+        self.layers: List[TobaraxLayer] = []
+        for i, L in enumerate(s.layers):
+            p = f"l{i}."
+            cls = MIXERS[L.mixer.kind]
+            rows = [mat(p + "mix." + n) for n in cls.IN]
+            cols = [mat(p + "mix.o")]
+            if L.ff is not None:
+                rows += [mat(p + "mlp.gate"), mat(p + "mlp.up")]
+                cols.append(mat(p + "mlp.down"))
+            self.layers.append(TobaraxLayer(
+                norm1=vec(p + "norm1"),
+                norm2=vec(p + "norm2") if L.ff is not None else None,
+                w_in=torch.cat(rows, dim=0).contiguous(),
+                w_out=torch.cat(cols, dim=1).contiguous(),
+                mixer=cls(L.mixer, s.norm_eps,
+                          lambda n, p=p: mat(p + "mix." + n),
+                          lambda n, p=p: vec(p + "mix." + n))))
+        self.norm_f = vec("final.norm")
+        self.lm_head = mat("head")
+        self.loop_in = mat("loop.in") if s.loop is not None else None
+        self.loop_step = vec("loop.step") if s.loop is not None else None
+
+    def load_weights(self, path: str) -> None:
+        self._set_weights(self._read(path))
+
+    def state_dict_full(self) -> Dict[str, torch.Tensor]:
+        """Tensors under their names in a model folder."""
+        s, out = self.spec, {"embed": self.emb, "head": self.lm_head,
+                             "final.norm": self.norm_f}
+        if s.loop is not None:
+            out["loop.in"], out["loop.step"] = self.loop_in, self.loop_step
+        for i, (L, lw) in enumerate(zip(s.layers, self.layers)):
+            p, m = f"l{i}.", L.mixer
+            out[p + "norm1"] = lw.norm1
+            shapes = lw.mixer.shapes(m, s.hidden_size)
+            at = 0
+            for n in lw.mixer.IN:
+                out[p + "mix." + n] = lw.w_in[at:at + shapes[n][0]]
+                at += shapes[n][0]
+            out[p + "mix.o"] = lw.w_out[:, :m.out_cols]
+            for n, t in lw.mixer.own_weights().items():
+                out[p + "mix." + n] = t
+            if L.ff is not None:
+                out[p + "norm2"] = lw.norm2
+                out[p + "mlp.gate"] = lw.w_in[at:at + L.ff]
+                out[p + "mlp.up"] = lw.w_in[at + L.ff:]
+                out[p + "mlp.down"] = lw.w_out[:, m.out_cols:]
+        return out
+
+    def save_weights(self, path: str) -> None:
+        """Write a model folder (bfloat16, as such folders are)."""
+        from safetensors.torch import save_file
+
+        os.makedirs(path, exist_ok=True)
+        save_file({k: v.to(torch.bfloat16).contiguous().cpu()
+                   for k, v in self.state_dict_full().items()},
+                  os.path.join(path, "model.safetensors"))
+        with open(os.path.join(path, "config.json"), "w",
+                  encoding="utf-8") as f:
+            json.dump(self.spec.to_config(), f, indent=1)
+
+    def param_bytes(self) -> int:
+        return sum(t.numel() * t.element_size()
+                   for t in self.state_dict_full().values())
+
+    # -- cache -----------------------------------------------------------------
+
+    def new_cache(self, num_blocks: int, num_slots: int,
+                  block_size: int = 64) -> HybridCache:
+        mixers = [self.layers[r.layer].mixer for r in self.spec.runs]
+        return HybridCache(
+            [m.row_width for m in mixers], [m.state_shape for m in mixers],
+            num_blocks, num_slots, block_size, self.device, self.dtype)
+
+    def cache_bytes_per_token(self) -> int:
+        el = torch.empty(0, dtype=self.dtype).element_size()
+        return el * sum(self.layers[r.layer].mixer.row_width or 0
+                        for r in self.spec.runs)
+
+    # -- forward -----------------------------------------------------------------
+
+    def forward(self, batch, cache: HybridCache,
+                on_run: Optional[Callable[[int, torch.Tensor], None]] = None
+                ) -> torch.Tensor:
+        """One step -> float32 logits of ``batch.want_rows`` (all rows if
+        None). ``on_run(r, residual)`` is called after every layer run."""
+        s, dt = self.spec, self.dtype
+        x = torch.nn.functional.embedding(batch.tokens, self.emb).float()
+        x0 = x.clone() if s.loop is not None else None
+        for r, run in enumerate(s.runs):
+            if run.enters_pass is not None:
+                x = ops.linear_f32(ops.cat_cast(x, x0, dt), self.loop_in,
+                                   self.loop_step[run.enters_pass])
+            lw, L = self.layers[run.layer], s.layers[run.layer]
+            n1, n2 = ops.norm_pair(x, lw.norm1, lw.norm2, s.norm_eps, dt)
+            n_mix, ff = L.mixer.out_cols, L.ff or 0
+            cat = torch.empty(x.shape[0], n_mix + ff, dtype=dt,
+                              device=x.device)
+            proj = ops.mix_in(n1, n2, lw.w_in, L.mixer.in_rows, ff,
+                              cat[:, n_mix:])
+            lw.mixer.run(proj, cat[:, :n_mix], batch, cache, r, self._rot)
+            x = ops.residual_linear(x, cat, lw.w_out)
+            if on_run is not None:
+                on_run(r, x)
+        if batch.want_rows is not None:
+            x = x[batch.want_rows]
+        y, _ = ops.norm_pair(x, self.norm_f, None, s.norm_eps, dt)
+        return ops.logits_head(y, self.lm_head, s.logit_scale,
+                               s.logit_softcap)

@@ -19,7 +19,12 @@ from typing import Optional, Tuple
 
 import torch
 
+from fei_amd.ops import mixers as _mixers
 from fei_amd.ops import reference as ref
+from fei_amd.ops.mixers import (  # noqa: F401
+    cat_cast, check_gla_geometry, check_latent_geometry, gla_decode,
+    gla_prefill, latent_attn_decode, latent_attn_prefill, linear_f32,
+    logits_head, mix_in, norm_pair, residual_linear)
 
 _LIB: Optional[ctypes.CDLL] = None
 _LIB_ERR: Optional[str] = None
@@ -89,6 +94,7 @@ def _try_load() -> None:
                                   _vp]
     lib.fei_gemv_swiglu_norm.argtypes = [_vp, _vp, _vp, _vp, _i, _i, _i, _f,
                                          _i, _vp, _vp]
+    _mixers.declare(lib)
     _LIB = lib
 
 
@@ -106,6 +112,16 @@ def require_lib() -> ctypes.CDLL:
             "`python -m fei_amd.ops.build` — GPU execution refuses to fall "
             "back to eager PyTorch.")
     return _LIB
+
+
+def build_if_missing() -> None:
+    """Compile the kernel library if this checkout has none (or an older
+    one); needs hipcc, takes about a minute."""
+    global _LIB_ERR
+    from fei_amd.ops import build as _build
+    if _build.needs_build():
+        _build.build(verbose=False)
+        _LIB_ERR = None
 
 
 def _stream() -> int:

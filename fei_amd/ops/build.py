@@ -15,7 +15,9 @@ from concurrent.futures import ThreadPoolExecutor
 
 CSRC = os.path.join(os.path.dirname(os.path.abspath(__file__)), "csrc")
 OUT = os.path.join(os.path.dirname(os.path.abspath(__file__)), "libfei_kernels.so")
-SOURCES = ["fei_kernels.hip", "attn_prefill.hip", "gemv.hip", "attn_decode_fused.hip", "gemv_fp8.hip", "stream_layer.hip"]
+SOURCES = ["fei_kernels.hip", "attn_prefill.hip", "gemv.hip", "attn_decode_fused.hip", "gemv_fp8.hip", "stream_layer.hip",
+           "hybrid.hip", "latent_attn.hip", "gla.hip"]
+HEADERS = ["fei_common.h", "fei_epilogue.h", "fei_mma.h"]
 HIPCC = os.environ.get("HIPCC", "hipcc")
 ARCH = os.environ.get("FEI_AMD_ARCH", "gfx950")
 # Packed fp32 VALU instructions are off: some of their forms have returned
@@ -28,7 +30,7 @@ def needs_build() -> bool:
     if not os.path.exists(OUT):
         return True
     out_mtime = os.path.getmtime(OUT)
-    for src in SOURCES + ["fei_common.h"]:
+    for src in SOURCES + HEADERS:
         if os.path.getmtime(os.path.join(CSRC, src)) > out_mtime:
             return True
     return False

@@ -14,6 +14,7 @@
 // (rows n and n+N) and writes silu(g)*u — kills the separate swiglu
 // kernel and the 2*I-wide intermediate.
 #include "fei_common.h"
+#include "fei_epilogue.h"
 
 namespace {
 
@@ -453,10 +454,10 @@ namespace {
 
 typedef __attribute__((ext_vector_type(4))) float f32x4_g;
 
-template <bool NTW>
+template <bool NTW, int EPI>
 __global__ void __launch_bounds__(256)
-k_gemm_m8(u16* __restrict__ out, const u16* __restrict__ x,
-          const u16* __restrict__ w, int M, int N, int K) {
+k_gemm_m8(void* __restrict__ outp, const u16* __restrict__ x,
+          const u16* __restrict__ w, int M, int N, int K, Epilogue ep) {
   const int n0 = blockIdx.x * GEMM_NT;
   const int tid = threadIdx.x;
   const int wv = tid >> 6;
@@ -511,21 +512,39 @@ k_gemm_m8(u16* __restrict__ out, const u16* __restrict__ x,
       const int m = i / 16, n = i % 16;
       const float v = cred[0][m][n] + cred[1][m][n] + cred[2][m][n] +
                       cred[3][m][n];
-      out[(long)m * N + n0 + n] = f2bf(v);
+      epilogue<EPI>(outp, (long)m * N + n0 + n, n0 + n, v, ep);
     }
   }
 }
 
 }  // namespace
 
+// float32 results: residual != 0 adds to out, otherwise out is
+// softcap(acc * scale, cap) + bias (cap 0: none; bias may be null).
+extern "C" void fei_gemm_m8_f32(void* out, const void* x, const void* w,
+                                const float* bias, int M, int N, int K,
+                                int residual, float scale, float cap,
+                                hipStream_t stream) {
+  dim3 grid(N / GEMM_NT);
+  const Epilogue ep{bias, scale, cap};
+  if (residual)
+    hipLaunchKernelGGL((k_gemm_m8<false, EPI_RES>), grid, dim3(256), 0, stream,
+                       out, (const u16*)x, (const u16*)w, M, N, K, ep);
+  else
+    hipLaunchKernelGGL((k_gemm_m8<false, EPI_F32>), grid, dim3(256), 0, stream,
+                       out, (const u16*)x, (const u16*)w, M, N, K, ep);
+}
+
 extern "C" void fei_gemm_m8(void* out, const void* x, const void* w, int M,
                             int N, int K, int nontemporal,
                             hipStream_t stream) {
   dim3 grid(N / GEMM_NT);
   if (nontemporal)
-    hipLaunchKernelGGL(k_gemm_m8<true>, grid, dim3(256), 0, stream,
-                       (u16*)out, (const u16*)x, (const u16*)w, M, N, K);
+    hipLaunchKernelGGL((k_gemm_m8<true, EPI_BF16>), grid, dim3(256), 0,
+                       stream, out, (const u16*)x, (const u16*)w, M, N, K,
+                       Epilogue{});
   else
-    hipLaunchKernelGGL(k_gemm_m8<false>, grid, dim3(256), 0, stream,
-                       (u16*)out, (const u16*)x, (const u16*)w, M, N, K);
+    hipLaunchKernelGGL((k_gemm_m8<false, EPI_BF16>), grid, dim3(256), 0,
+                       stream, out, (const u16*)x, (const u16*)w, M, N, K,
+                       Epilogue{});
 }

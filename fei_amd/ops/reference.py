@@ -274,3 +274,106 @@ def hash_gumbel(B: int, v_local: int, v_offset: int, seed: int,
             out[b] = (m + 1.0) * (1.0 / 16777216.0)
     u = torch.from_numpy(out)
     return -torch.log(-torch.log(u))
+
+
+# -- ops of decoders made of unlike layers -------------------------------------
+# Rows are flat [T, C]: the tokens of several sequences one after another. The
+# residual, norms, angles, scores and recurrences are float32; projections and
+# cached rows have the model's dtype.
+
+def rope_table_exact(max_seq: int, dim: int, base: float,
+                     device=None) -> torch.Tensor:
+    """[max_seq, dim/2, 2] cos/sin of p * base^(-2i/dim), each rounded once
+    from float64."""
+    inv = base ** (-torch.arange(0, dim, 2, dtype=torch.float64) / max(dim, 1))
+    ang = torch.outer(torch.arange(max_seq, dtype=torch.float64), inv)
+    return torch.stack([ang.cos(), ang.sin()], dim=-1).float().contiguous() \
+        .to(device)
+
+
+def apply_rope_interleaved(x: torch.Tensor, positions: torch.Tensor,
+                           table: torch.Tensor) -> torch.Tensor:
+    """x [T, ..., D] float32, pairs (2i, 2i+1); positions [T]."""
+    cs = table[positions.long()]
+    shape = [x.shape[0]] + [1] * (x.dim() - 2) + [x.shape[-1] // 2]
+    cos, sin = cs[..., 0].reshape(shape), cs[..., 1].reshape(shape)
+    u, v = x[..., 0::2].float(), x[..., 1::2].float()
+    return torch.stack([u * cos - v * sin, v * cos + u * sin], dim=-1) \
+        .flatten(-2)
+
+
+def rms(x: torch.Tensor, eps: float) -> torch.Tensor:
+    xf = x.float()
+    return xf * torch.rsqrt(xf.pow(2).mean(dim=-1, keepdim=True) + eps)
+
+
+def norm_pair(x, w1, w2, eps, dtype):
+    """Two weighted RMS norms of the same rows."""
+    y = rms(x, eps)
+    return (y * w1).to(dtype), None if w2 is None else (y * w2).to(dtype)
+
+
+def softcap_logits(y: torch.Tensor, scale: float,
+                   cap: Optional[float]) -> torch.Tensor:
+    y = y.float() * scale
+    return y if cap is None else cap * torch.tanh(y / cap)
+
+
+def latent_append(proj, m, norm_w, rot, eps, pos, dst, rows):
+    """Latent (normed) and rotated key part of each row of ``proj``, into
+    ``rows[dst]``; returns the rotated queries, float32 [T, H, dim+rot_dim]."""
+    nq = m.heads * (m.dim + m.rot_dim)
+    c = rms(proj[:, nq:nq + m.kv_rank], eps) * norm_w
+    kr = proj[:, nq + m.kv_rank:nq + m.row_width].float()
+    q = proj[:, :nq].float().view(-1, m.heads, m.dim + m.rot_dim).clone()
+    if m.rot_dim:
+        kr = apply_rope_interleaved(kr, pos, rot)
+        q[..., m.dim:] = apply_rope_interleaved(
+            q[..., m.dim:].contiguous(), pos, rot)
+    rows[dst.long()] = torch.cat([c, kr], dim=-1).to(rows.dtype)
+    return q
+
+
+def latent_attend(q, pos, keys, k0, m, uk, uv, scale):
+    """q [n, H, dim+rot_dim] at positions ``pos`` [n]; keys [N, row_width]
+    cached rows of positions k0 .. k0+N-1. Returns [n, H, vdim]."""
+    H, N = m.heads, keys.shape[0]
+    c, kr = keys[:, :m.kv_rank].float(), keys[:, m.kv_rank:].float()
+    k = torch.nn.functional.linear(c, uk.float()).view(N, H, m.dim)
+    v = torch.nn.functional.linear(c, uv.float()).view(N, H, m.vdim)
+    s = torch.einsum("nhd,khd->hnk", q[..., :m.dim], k)
+    if m.rot_dim:
+        s = s + torch.einsum("nhd,kd->hnk", q[..., m.dim:], kr)
+    s = s * scale
+    kp = torch.arange(k0, k0 + N, device=q.device).view(1, 1, N)
+    qp = pos.long().view(1, -1, 1)
+    hide = kp > qp
+    if m.window is not None:
+        hide = hide | (qp - kp >= m.window)
+    p = torch.softmax(s.masked_fill(hide, float("-inf")), dim=-1)
+    return torch.einsum("hnk,khd->nhd", p, v)
+
+
+def gla_log_decay(a1, a2, bias, tau):
+    """log of sigmoid(z)^(1/tau), z = a2 a1 + bias; float32 [T, H*dim]."""
+    z = torch.nn.functional.linear(a1.float(), a2.float()) + bias
+    return torch.nn.functional.logsigmoid(z) / tau
+
+
+def gla_scan(q, k, v, logdecay, state):
+    """q, k, logdecay [T, H, d], v [T, H, e], state [H, e, d] (float32),
+    token by token. Returns o [T, H, e] and the last state."""
+    out = torch.empty(q.shape[0], q.shape[1], v.shape[-1])
+    S = state.clone()
+    decay = logdecay.exp()
+    for t in range(q.shape[0]):
+        S = S * decay[t].unsqueeze(1) + v[t].unsqueeze(-1) * k[t].unsqueeze(1)
+        out[t] = (S * q[t].unsqueeze(1)).sum(-1)
+    return out, S
+
+
+def gla_gate_out(o, g, norm_w, eps):
+    """Per-head RMS norm of o [T, H, e], times silu(g) [T, H*e]."""
+    y = (rms(o, eps) * norm_w).flatten(1)
+    gf = g.float()
+    return y * (gf * torch.sigmoid(gf))
