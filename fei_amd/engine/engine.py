@@ -28,9 +28,10 @@ from typing import Dict, List, Optional, Union
 import torch
 
 from fei_amd import ops
-from fei_amd.engine.config import ModelSpec, get_spec
+from fei_amd.engine.config import AnySpec, MODEL_SPECS, get_spec, is_model_folder
+from fei_amd.engine.step import StepEntry, StepRunner
 from fei_amd.engine.tokenizer import ByteTokenizer
-from fei_amd.models.llama import LlamaModel
+from fei_amd.models import model_class
 from fei_amd.parallel.pg import ParallelContext
 from fei_amd.utils.logging import get_logger
 
@@ -42,7 +43,7 @@ SAMPLE_CHUNKS = 64       # stage-1 blocks for the sampling kernel
 class LocalEngine:
     def __init__(
         self,
-        spec: ModelSpec,
+        spec: AnySpec,
         device: Optional[torch.device] = None,
         batch_size: int = 1,
         max_seq_len: Union[int, str, None] = None,   # int | "hbm" | None
@@ -54,6 +55,8 @@ class LocalEngine:
         weight_quant: Optional[str] = None,    # None | "fp8" (decode path)
         tokenizer=None,                        # default ByteTokenizer; or
                                                # SpmTokenizer(model_path)
+        weights: Optional[str] = None,         # model folder; default the
+                                               # FEI_WEIGHTS env, else random
     ):
         self.spec = spec
         if device is None:
@@ -150,30 +153,50 @@ class LocalEngine:
                 2 * spec.num_layers * spec.hidden_size *
                 spec.intermediate_size * 12 // 10 ** 9)
         t0 = time.perf_counter()
-        self.model = LlamaModel(spec, device, dtype, tp=self.tp, seed=seed,
-                                max_seq_len=self.max_seq_len)
-        w_path = _os.environ.get("FEI_WEIGHTS")
+        cls = model_class(spec)
+        w_path = weights or _os.environ.get("FEI_WEIGHTS")
+        at_once = {"weights": w_path} if getattr(cls, "step_cache", False) \
+            else {}
+        t1 = time.perf_counter()
+        self.model = cls(spec, device, dtype, tp=self.tp, seed=seed,
+                         max_seq_len=self.max_seq_len, **at_once)
+        # models of unlike layers run through a StepRunner and its cache;
+        # the others have one contiguous KV cache per layer
+        self.step_cache = getattr(self.model, "step_cache", False)
+        # a recurrent state holds exactly the tokens it has read: it can go
+        # on from there, but not from an earlier position
+        self.recurrent = getattr(self.model, "recurrent", False)
         if w_path:
-            t1 = time.perf_counter()
-            self.model.load_weights(w_path)
+            if not at_once:
+                t1 = time.perf_counter()
+                self.model.load_weights(w_path)
             logger.info("loaded weights from %s in %.1fs", w_path,
                         time.perf_counter() - t1)
         if self._hbm_seq:
             self.max_seq_len = self._resolve_hbm_seq()
             # RoPE table must cover the enlarged window
-            from fei_amd.ops import reference as _ref
-            self.model.max_seq_len = self.max_seq_len
-            self.model.rope = _ref.rope_table(
-                self.max_seq_len, self.model.D, spec.rope_theta,
-                device=device)
+            self.model.resize(self.max_seq_len)
             logger.info("max_seq_len='hbm' -> %d tokens (%.1f GB KV)",
                         self.max_seq_len,
                         self._kv_bytes_per_token() * self.B *
                         self.max_seq_len / 2 ** 30)
-        self.k_caches, self.v_caches = self.model.new_kv_cache(self.B, self.max_seq_len)
+        if self.step_cache:
+            per_seq = -(-self.max_seq_len // 64)
+            self.runner: Optional[StepRunner] = StepRunner(
+                self.model, num_blocks=self.B * per_seq, num_slots=self.B)
+            self._seqs = [self.runner.admit(self.max_seq_len)
+                          for _ in range(self.B)]
+            self.k_caches, self.v_caches = [], []
+        else:
+            self.runner = None
+            self.k_caches, self.v_caches = self.model.new_kv_cache(
+                self.B, self.max_seq_len)
         logger.info("model %s init in %.1fs (%.2f GB params)", spec.name,
                     time.perf_counter() - t0, self.model.param_bytes() / 2**30)
         self.weight_quant = weight_quant or _os.environ.get("FEI_WEIGHT_QUANT")
+        if self.step_cache and self.weight_quant:
+            raise ValueError(f"{spec.name}: weight quantization is not "
+                             "available for this architecture")
         if self._fused_norm_env is not None:
             self.fused_norm = self._fused_norm_env not in ("0", "false")
         else:
@@ -193,22 +216,13 @@ class LocalEngine:
                                       dtype=torch.int32, device=device)
         self.sample_ws = torch.zeros(self.B, SAMPLE_CHUNKS, 2,
                                      dtype=torch.float32, device=device)
-        Hq_l, D = self.model.hq_l, self.model.D
-        # sized from self.attn_splits (NOT the ctor arg: FEI_ATTN_SPLITS
-        # overrides it, and an undersized workspace is an out-of-bounds
-        # write in the split kernel)
-        # 3rd element: zeroed per-split done-flag buffer [B*Hkv_l*splits]
-        # selecting the FUSED split-K combine (split 0 of each (b, hkv)
-        # pair polls the flags and reduces the partials in-kernel — no
-        # separate combine launch per layer).
-        self.attn_ws = (
-            torch.zeros(self.B, Hq_l, self.attn_splits, D, dtype=torch.float32, device=device),
-            torch.zeros(self.B, Hq_l, self.attn_splits, 2, dtype=torch.float32, device=device),
-            torch.zeros(self.B * self.model.hkv_l * self.attn_splits,
-                        dtype=torch.int32, device=device),
-        )
-        self.attn_out = torch.zeros(self.B, Hq_l, D, dtype=self.dtype,
-                                    device=device)
+        self.attn_ws = ()
+        if self.step_cache:
+            self.batch = self.runner.decode_batch(self._seqs,
+                                                  room=self.max_seq_len)
+            self.batch.tokens, self.batch.pos = self.token, self.pos
+        else:
+            self._init_attn_ws()
         # Persistent weight-streaming decode engine (FEI_STREAM_DECODE=1):
         # one launch per layer on the LDS-DMA loader/consumer structure
         # (ops/csrc/stream_layer.hip) instead of six. Guarded by the
@@ -254,9 +268,30 @@ class LocalEngine:
             torch.nn.functional.linear(a, w)
             torch.cuda.synchronize(device)
 
+    def _init_attn_ws(self) -> None:
+        device = self.device
+        Hq_l, D = self.model.hq_l, self.model.D
+        # sized from self.attn_splits (NOT the ctor arg: FEI_ATTN_SPLITS
+        # overrides it, and an undersized workspace is an out-of-bounds
+        # write in the split kernel)
+        # 3rd element: zeroed per-split done-flag buffer [B*Hkv_l*splits]
+        # selecting the FUSED split-K combine (split 0 of each (b, hkv)
+        # pair polls the flags and reduces the partials in-kernel — no
+        # separate combine launch per layer).
+        self.attn_ws = (
+            torch.zeros(self.B, Hq_l, self.attn_splits, D, dtype=torch.float32, device=device),
+            torch.zeros(self.B, Hq_l, self.attn_splits, 2, dtype=torch.float32, device=device),
+            torch.zeros(self.B * self.model.hkv_l * self.attn_splits,
+                        dtype=torch.int32, device=device),
+        )
+        self.attn_out = torch.zeros(self.B, Hq_l, D, dtype=self.dtype,
+                                    device=device)
+
     # -- construction helpers ------------------------------------------------
 
     def _kv_bytes_per_token(self) -> int:
+        if self.step_cache:
+            return self.model.cache_bytes_per_token()
         s = self.spec
         el = 2 if self.dtype == torch.bfloat16 else 4
         return (s.num_layers * (s.num_kv_heads //
@@ -279,11 +314,27 @@ class LocalEngine:
         return int(seq)
 
     @classmethod
-    def create(cls, model: Union[str, ModelSpec] = "llama3-8b", **kwargs) -> "LocalEngine":
+    def create(cls, model: Union[str, AnySpec] = "llama3-8b", **kwargs) -> "LocalEngine":
+        """``model``: a registered name, a model folder (config.json +
+        model.safetensors, whose weights are loaded), or a spec."""
         spec = get_spec(model) if isinstance(model, str) else model
+        if isinstance(model, str) and model not in MODEL_SPECS \
+                and is_model_folder(model):
+            kwargs.setdefault("weights", model)
         return cls(spec, **kwargs)
 
     # -- decode step ---------------------------------------------------------
+
+    def _decode_logits(self) -> torch.Tensor:
+        """Logits of one decode step of every row, at self.pos."""
+        if self.step_cache:
+            with torch.no_grad():
+                return self.model.forward(self.batch, self.runner.cache)
+        return self.model.forward_decode(
+            self.token, self.pos, self.k_caches, self.v_caches,
+            attn_splits=self.attn_splits, workspace=self.attn_ws,
+            fused_attn=self.fused_attn, attn_out=self.attn_out,
+            fused_norm=self.fused_norm)
 
     def _decode_step(self) -> None:
         if self.tp.is_distributed:
@@ -299,11 +350,7 @@ class LocalEngine:
                        nchunks=SAMPLE_CHUNKS)
             ops.advance(self.pos, self.step, max_pos=self.max_seq_len - 1)
             return
-        logits = self.model.forward_decode(
-            self.token, self.pos, self.k_caches, self.v_caches,
-            attn_splits=self.attn_splits, workspace=self.attn_ws,
-            fused_attn=self.fused_attn, attn_out=self.attn_out,
-            fused_norm=self.fused_norm)
+        logits = self._decode_logits()
         ops.sample(logits, self.token, self.step, self.sample_ws.view(self.B, -1),
                    out_tokens=self.out_tokens, temperature=self.temperature,
                    seed=self.seed, nchunks=SAMPLE_CHUNKS)
@@ -354,6 +401,13 @@ class LocalEngine:
             "step": self.step.clone(),
             "out": self.out_tokens[:, :4].clone(),
         }
+        # a step cache has a block and a slot for this: the warmup runs
+        # there and touches no sequence
+        if self.step_cache:
+            saved["table"] = self.batch.table.clone()
+            saved["slots"] = self.batch.slots.clone()
+            self.batch.table.fill_(self.runner.cache.scratch_block)
+            self.batch.slots.fill_(self.runner.cache.scratch_slot)
         # warmup at positions 1..2: snapshot those KV rows in every layer
         kv_rows = slice(1, 4)
         saved_k = [k[:, :, kv_rows].clone() for k in self.k_caches]
@@ -376,6 +430,9 @@ class LocalEngine:
         self.pos.copy_(saved["pos"])
         self.step.copy_(saved["step"])
         self.out_tokens[:, :4].copy_(saved["out"])
+        if self.step_cache:
+            self.batch.table.copy_(saved["table"])
+            self.batch.slots.copy_(saved["slots"])
         for k, sk in zip(self.k_caches, saved_k):
             k[:, :, kv_rows].copy_(sk)
         for v, sv in zip(self.v_caches, saved_v):
@@ -423,6 +480,39 @@ class LocalEngine:
 
     PREFILL_CHUNK = 2048      # bounds activation memory for long prompts
 
+    def _prefill_logits(self, rows: List[List[int]], from_pos: int,
+                        all_positions: bool = False) -> torch.Tensor:
+        """Run ``rows`` (sequences 0 .. len(rows)-1, equally long) from
+        position ``from_pos``: logits of the last position [n, V], or of all
+        [n, S, V]."""
+        if not self.step_cache:
+            tokens = torch.tensor(rows, dtype=torch.int64, device=self.device)
+            pos0 = torch.full((len(rows),), from_pos, dtype=torch.int32,
+                              device=self.device)
+            return self.model.forward_prefill(
+                tokens, pos0, self.k_caches, self.v_caches,
+                all_positions=all_positions)
+        for sid in self._seqs[:len(rows)]:
+            if self.recurrent and from_pos not in (0, self.runner.length[sid]):
+                raise ValueError("a recurrent state cannot go back to "
+                                 f"position {from_pos}")
+            self.runner.set_length(sid, from_pos)
+        S = len(rows[0])
+        want = range(S) if all_positions else [S - 1]
+        logits = self.runner.step([StepEntry(sid, r, want)
+                                   for sid, r in zip(self._seqs, rows)])
+        return logits.view(len(rows), S, -1) if all_positions else logits
+
+    def _sampled_dtype(self, logits: torch.Tensor) -> torch.Tensor:
+        """A step model's float32 logits are sampled as they are."""
+        return logits if self.step_cache else logits.to(self.dtype)
+
+    def _sync_runner(self) -> None:
+        """Decoding advances ``pos`` on the device: tell the runner."""
+        if self.step_cache:
+            for sid, p in zip(self._seqs, self.pos.tolist()):
+                self.runner.set_length(sid, p)
+
     def prefill(self, token_ids: List[int], from_pos: int = 0) -> None:
         """Prefill ``token_ids`` starting at cache position ``from_pos``
         (0 = fresh conversation; >0 = prefix-cache extension: the first
@@ -451,27 +541,19 @@ class LocalEngine:
             budget = self.max_seq_len - 1
         if len(token_ids) > budget:
             token_ids = token_ids[-budget:]
+        if from_pos:
+            self._sync_runner()
         while len(token_ids) > self.PREFILL_CHUNK:
             head, token_ids = (token_ids[:self.PREFILL_CHUNK],
                                token_ids[self.PREFILL_CHUNK:])
-            tokens = torch.tensor([head] * self.B, dtype=torch.int64,
-                                  device=self.device)
-            pos0 = torch.full((self.B,), from_pos, dtype=torch.int32,
-                              device=self.device)
-            self.model.forward_prefill(tokens, pos0, self.k_caches,
-                                       self.v_caches)
+            self._prefill_logits([head] * self.B, from_pos)
             from_pos += len(head)
         S = len(token_ids)
         self.ensure_graph()
-        tokens = torch.tensor([token_ids] * self.B, dtype=torch.int64,
-                              device=self.device)
-        pos0 = torch.full((self.B,), from_pos, dtype=torch.int32,
-                          device=self.device)
-        logits = self.model.forward_prefill(tokens, pos0, self.k_caches,
-                                            self.v_caches)
+        logits = self._prefill_logits([token_ids] * self.B, from_pos)
         self.step.zero_()
         self.out_tokens.zero_()
-        ops.sample(logits.to(self.dtype), self.token, self.step,
+        ops.sample(self._sampled_dtype(logits), self.token, self.step,
                    self.sample_ws.view(self.B, -1), out_tokens=self.out_tokens,
                    temperature=self.temperature, seed=self.seed,
                    nchunks=SAMPLE_CHUNKS)
@@ -544,6 +626,10 @@ class LocalEngine:
 
         assert self.B == 1, "speculative decode is a batch-1 agent path"
         assert self.temperature == 0.0, "speculative decode is greedy-only"
+        if self.recurrent:
+            raise ValueError("speculative decode needs a cache that can drop "
+                             "rejected tokens; a recurrent state cannot")
+        self._sync_runner()
         eos = self.tokenizer.eos_id
         first = int(self.token[0])            # token sampled by prefill
         index = NgramIndex()
@@ -561,11 +647,7 @@ class LocalEngine:
                 L = len(block)
                 if L == 0:
                     break
-            tokens = torch.tensor([block], dtype=torch.int64, device=self.device)
-            pos0 = torch.full((1,), pos_h, dtype=torch.int32, device=self.device)
-            logits = self.model.forward_prefill(tokens, pos0, self.k_caches,
-                                                self.v_caches,
-                                                all_positions=True)
+            logits = self._prefill_logits([block], pos_h, all_positions=True)
             greedy = logits[0].argmax(dim=-1).tolist()        # len L
             n_acc = 0
             while n_acc < len(props) and props[n_acc] == greedy[n_acc]:
@@ -625,7 +707,8 @@ class LocalEngine:
             import os as _os
             speculative = _os.environ.get("FEI_SPEC_DECODE", "0") == "1"
         spec_metrics: Dict[str, object] = {}
-        if speculative and self.B == 1 and temperature == 0.0:
+        if speculative and self.B == 1 and temperature == 0.0 \
+                and not self.recurrent:
             ctx = prompt_ids[:from_pos] + new_ids
             self.last_metrics = {}
             rows = self.decode_speculative(max_new_tokens, ctx,
@@ -675,6 +758,11 @@ class LocalEngine:
         if from_pos > len(prompt_ids):
             from_pos = 0
         new_ids = prompt_ids[from_pos:]
+        if from_pos and self.recurrent and from_pos != int(self.pos[0]):
+            # the state covers more (or fewer) tokens than the shared prefix
+            from_pos, new_ids = 0, prompt_ids
+        if not new_ids and self.recurrent:
+            from_pos, new_ids = 0, prompt_ids
         if not new_ids:                      # identical prompt: redo last token
             from_pos = max(0, len(prompt_ids) - 1)
             new_ids = prompt_ids[from_pos:]
@@ -775,11 +863,9 @@ class LocalEngine:
             return {"logprob": 0.0, "token_logprobs": [], "is_greedy": True}
         ids = (ctx + cont)[-(self.max_seq_len - 1):]
         n_cont = min(len(cont), len(ids) - 1)
-        tokens = torch.tensor([ids], dtype=torch.int64, device=self.device)
-        pos0 = torch.zeros(1, dtype=torch.int32, device=self.device)
-        logits = self.model.forward_prefill(tokens, pos0, self.k_caches,
-                                            self.v_caches,
-                                            all_positions=True)[0].float()
+        logits = self._prefill_logits([ids], 0, all_positions=True)[0].float()
+        if self.recurrent:
+            self.pos.zero_()         # no prefix to continue from any more
         # logits[i] predicts ids[i+1]
         lp = torch.log_softmax(logits[:-1], dim=-1)
         start = len(ids) - 1 - n_cont
@@ -793,7 +879,7 @@ class LocalEngine:
 
     def shutdown(self) -> None:
         self._graph = None
-        self.k_caches = self.v_caches = None  # release HBM
+        self.k_caches = self.v_caches = self.runner = None  # release HBM
         if self.is_gpu:
             torch.cuda.empty_cache()
 
@@ -805,12 +891,7 @@ class LocalEngine:
         path covers greedy + plain Gumbel; filtered sampling runs eagerly)."""
         from fei_amd.ops import reference as ref
 
-        logits = self.model.forward_decode(
-            self.token, self.pos, self.k_caches, self.v_caches,
-            attn_splits=self.attn_splits, workspace=self.attn_ws,
-            fused_attn=self.fused_attn, attn_out=self.attn_out,
-            fused_norm=self.fused_norm)
-        masked = logits.float()
+        masked = self._decode_logits().float()
         if top_k:
             masked = ref.topk_mask(masked, top_k)
         if top_p < 1.0:
@@ -859,6 +940,30 @@ class LocalEngine:
         prompts = [p[-n:] if n < len(p) else p for p, n in zip(prompts, lens)]
         S = max(lens)
         self.ensure_graph()
+        if self.step_cache:
+            for sid in self._seqs:
+                self.runner.set_length(sid, 0)
+            logits = self.runner.step([StepEntry(sid, p, [len(p) - 1])
+                                       for sid, p in zip(self._seqs, prompts)])
+        else:
+            logits = self._prefill_padded(prompts, lens, S)
+        self.step.zero_()
+        self.out_tokens.zero_()
+        ops.sample(self._sampled_dtype(logits).contiguous(), self.token,
+                   self.step, self.sample_ws.view(self.B, -1),
+                   out_tokens=self.out_tokens,
+                   temperature=self.temperature, seed=self.seed,
+                   nchunks=SAMPLE_CHUNKS)
+        self.pos.copy_(torch.tensor(lens, dtype=torch.int32,
+                                    device=self.device))
+        if self.is_gpu:
+            torch.cuda.synchronize(self.device)
+            self.step.fill_(1)
+        else:
+            self.step += 1
+
+    def _prefill_padded(self, prompts, lens, S: int) -> torch.Tensor:
+        """Last-position logits of B prompts of unequal length."""
         tok = self.tokenizer
         padded = torch.full((self.B, S), tok.pad_id, dtype=torch.int64,
                             device=self.device)
@@ -869,20 +974,7 @@ class LocalEngine:
         all_logits = self.model.forward_prefill(
             padded, pos0, self.k_caches, self.v_caches, all_positions=True)
         idx = torch.tensor([n - 1 for n in lens], device=self.device)
-        logits = all_logits[torch.arange(self.B, device=self.device), idx]
-        self.step.zero_()
-        self.out_tokens.zero_()
-        ops.sample(logits.to(self.dtype).contiguous(), self.token, self.step,
-                   self.sample_ws.view(self.B, -1), out_tokens=self.out_tokens,
-                   temperature=self.temperature, seed=self.seed,
-                   nchunks=SAMPLE_CHUNKS)
-        self.pos.copy_(torch.tensor(lens, dtype=torch.int32,
-                                    device=self.device))
-        if self.is_gpu:
-            torch.cuda.synchronize(self.device)
-            self.step.fill_(1)
-        else:
-            self.step += 1
+        return all_logits[torch.arange(self.B, device=self.device), idx]
 
     def generate_batch(self, prompts, max_new_tokens: int = 256,
                        temperature: float = 0.0, stop_on_eos: bool = True):

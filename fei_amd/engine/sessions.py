@@ -12,6 +12,11 @@ microseconds of torch indexing per layer); the O(context) work — attention
 over the pool — is the paged HIP kernel, and all GEMVs take the same
 streaming kernels as the single-session path. Greedy decode (serving
 agents at temperature 0); graphs are off (batch membership changes).
+
+Models of unlike layers (``model.step_cache``) get ``StepSessionManager``, a
+subclass with the same surface whose steps are ragged batches: portions of
+prompts run beside the decoding sessions' tokens, so a long prompt does not
+stall the others.
 """
 
 from __future__ import annotations
@@ -29,6 +34,7 @@ import torch.nn.functional as F
 
 from fei_amd import ops
 from fei_amd.engine.kv_cache import PagedKVPool
+from fei_amd.engine.step import StepEntry, StepRunner
 from fei_amd.ops import reference as ref
 
 
@@ -43,6 +49,10 @@ class Session:
 
 
 class PagedSessionManager:
+    def __new__(cls, engine, *args, **kwargs):
+        step = getattr(engine.model, "step_cache", False)
+        return object.__new__(StepSessionManager if step else cls)
+
     def __init__(self, engine, block_size: int = 16,
                  num_blocks: Optional[int] = None,
                  mem_fraction: float = 0.25):
@@ -319,3 +329,135 @@ class PagedSessionManager:
                          else m.norm_f)
             x, h = ops.fused_add_rmsnorm(d, h, next_norm, s.norm_eps)
         return ops.linear_decode(x, m.lm_head)
+
+
+class StepSessionManager(PagedSessionManager):
+    """Sessions over a StepRunner: one cache of latent rows and state slots,
+    one ragged batch per step.
+
+    ``open`` admits a session (a state slot, and blocks for its prompt) and
+    queues its prompt. While any prompt is queued, a step takes the next token
+    of every decoding session and up to ``prefill_budget`` prompt tokens, in
+    order of admission; otherwise decoding runs in device-resident chunks.
+    """
+
+    def __init__(self, engine, block_size: int = 64,
+                 num_blocks: Optional[int] = None,
+                 mem_fraction: float = 0.25, max_sessions: int = 64,
+                 prefill_budget: int = 2048):
+        self.engine = engine
+        self.model = m = engine.model
+        if num_blocks is None:
+            if m.device.type == "cuda":
+                budget = int(torch.cuda.mem_get_info(m.device)[0] *
+                             mem_fraction)
+            else:
+                budget = 1 << 26
+            num_blocks = max(16, budget // max(
+                1, m.cache_bytes_per_token() * block_size))
+            # no more than all sessions at full length can use
+            num_blocks = min(num_blocks, max_sessions *
+                             -(-m.max_seq_len // block_size))
+        self.runner = StepRunner(m, num_blocks, max_sessions, block_size)
+        self.pool = self.runner.cache
+        self.prefill_budget = prefill_budget
+        self.sessions: Dict[int, Session] = {}
+        self.eos = engine.tokenizer.eos_id
+
+    # -- admission -----------------------------------------------------------
+
+    def open(self, prompt: Union[str, List[int]],
+             max_new_tokens: int = 256) -> int:
+        """Queue a session; MemoryError when no slot or blocks are free."""
+        ids = (self.engine.tokenizer.encode(prompt)
+               if isinstance(prompt, str) else list(prompt))
+        if not ids:
+            raise ValueError("empty prompt")
+        if len(ids) + 1 > self.model.max_seq_len:
+            raise ValueError(f"prompt of {len(ids)} tokens does not fit "
+                             f"{self.model.max_seq_len}")
+        sid = self.runner.admit(len(ids) + 1)
+        self.sessions[sid] = Session(sid=sid, prompt_ids=ids,
+                                     max_new_tokens=max_new_tokens)
+        return sid
+
+    def close(self, sid: int) -> None:
+        if self.sessions.pop(sid, None) is not None:
+            self.runner.release(sid)
+
+    # -- steps ---------------------------------------------------------------
+
+    def _emit(self, s: Session, token: int) -> None:
+        s.generated.append(token)
+        if token == self.eos or len(s.generated) >= s.max_new_tokens:
+            s.done = True
+
+    def _mixed_step(self, act: List[Session]) -> int:
+        """One ragged batch; sessions that took part."""
+        entries: List[StepEntry] = []
+        emits: List[Session] = []
+        budget = self.prefill_budget
+        for s in act:
+            n = len(s.prompt_ids)
+            if s.pos >= n:
+                entries.append(StepEntry(s.sid, [s.generated[-1]], [0]))
+                emits.append(s)
+            elif budget > 0:
+                part = s.prompt_ids[s.pos:s.pos + budget]
+                budget -= len(part)
+                last = s.pos + len(part) == n
+                entries.append(StepEntry(s.sid, part,
+                                         [len(part) - 1] if last else []))
+                if last:
+                    emits.append(s)
+        logits = self.runner.step(entries)
+        for e in entries:
+            self.sessions[e.seq].pos += len(e.tokens)
+        if emits:
+            for s, t in zip(emits, logits.argmax(dim=-1).tolist()):
+                self._emit(s, int(t))
+        return len(entries)
+
+    @torch.no_grad()
+    def step_chunk(self, chunk: int = 8) -> int:
+        """Up to ``chunk`` steps. Returns sessions advanced (0 = none)."""
+        advanced = 0
+        left = chunk
+        while left > 0:
+            for s in self.active:
+                if s.pos >= self.model.max_seq_len:
+                    s.done = True            # no room for another token
+            act = self.active
+            if not act:
+                break
+            if any(s.pos < len(s.prompt_ids) for s in act):
+                advanced = max(advanced, self._mixed_step(act))
+                left -= 1
+                continue
+            advanced = max(advanced, len(act))
+            left -= self._decode_chunk(act, left)
+        return advanced
+
+    def _decode_chunk(self, act: List[Session], chunk: int) -> int:
+        """Decode steps with token feedback on the device and one download. A
+        session that ends inside the chunk runs on to its end: its blocks and
+        slot are its own and go back when it is closed."""
+        n = min(chunk, min(self.model.max_seq_len - s.pos for s in act),
+                max(s.max_new_tokens - len(s.generated) for s in act))
+        batch = self.runner.decode_batch([s.sid for s in act], n,
+                                         [s.generated[-1] for s in act])
+        steps = []
+        for _ in range(n):
+            logits = self.model.forward(batch, self.runner.cache)
+            batch.tokens = logits.argmax(dim=-1)
+            batch.pos += 1
+            steps.append(batch.tokens)
+        rows = torch.stack(steps, dim=1).tolist()
+        for s, row in zip(act, rows):
+            self.runner.set_length(s.sid, s.pos + n)
+            for t in row:
+                if s.done:
+                    break
+                s.pos += 1
+                self._emit(s, int(t))
+        return n

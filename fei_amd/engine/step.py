@@ -119,9 +119,10 @@ class StepRunner:
         self.cache.release(sid)
         self.length.pop(sid, None)
 
-    def rewind(self, sid: int) -> None:
-        """Forget what a sequence has read; its blocks and slot stay."""
-        self.length[sid] = 0
+    def set_length(self, sid: int, n: int) -> None:
+        """The sequence's next token is at position ``n``: 0 to start over,
+        or what the caller ran on the device by itself."""
+        self.length[sid] = n
 
     # -- steps ---------------------------------------------------------------
 
@@ -204,7 +205,7 @@ class StepRunner:
                      tokens: Optional[Sequence[int]] = None) -> RaggedBatch:
         """A batch of one token per sequence whose ``tokens`` and ``pos`` the
         caller advances in place; blocks for ``room`` more tokens are
-        reserved. The caller reports what it ran with ``advance``."""
+        reserved. The caller reports what it ran with ``set_length``."""
         for s in seqs:
             if self.length[s] + room > self.model.max_seq_len:
                 raise ValueError("sequence longer than "
@@ -220,6 +221,3 @@ class StepRunner:
                              dtype=torch.int32, device=dev),
             row_seq=torch.arange(len(seqs), dtype=torch.int32, device=dev),
             table=table, slots=slots, n_dec=len(seqs))
-
-    def advance(self, sid: int, n: int) -> None:
-        self.length[sid] += n

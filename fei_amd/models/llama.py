@@ -63,8 +63,7 @@ class LlamaModel:
         self.vocab_l = spec.vocab_size // tp_size
         self.D = spec.head_dim
         self._init_weights(seed)
-        self.rope = ref.rope_table(self.max_seq_len, self.D, spec.rope_theta,
-                                   device=device)
+        self.resize(self.max_seq_len)
         # FEI_PREFETCH=<MB>: during each decode layer's attention window
         # (low HBM traffic) a side-stream kernel pre-reads the first MB of
         # that layer's gate/up weights into L2/L3 so the big GEMV partially
@@ -79,6 +78,12 @@ class LlamaModel:
         # atomics + block barrier + per-step zeroing cost ~84 us/step.
         # Kept opt-in for re-measurement on future silicon.
         self.norm_precomp = os.environ.get("FEI_NORM_PRECOMP", "0") == "1"
+
+    def resize(self, max_seq_len: int) -> None:
+        """Positions up to ``max_seq_len`` - 1 can be run from now on."""
+        self.max_seq_len = max_seq_len
+        self.rope = ref.rope_table(max_seq_len, self.D, self.spec.rope_theta,
+                                   device=self.device)
 
     # -- weights -------------------------------------------------------------
 

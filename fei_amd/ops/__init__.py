@@ -56,7 +56,7 @@ def _try_load() -> None:
     lib.fei_attn_decode_combine.argtypes = [_vp, _vp, _vp, _i, _i, _i, _i, _vp]
     lib.fei_swiglu.argtypes = [_vp, _vp, _l, _i, _vp]
     lib.fei_sample.argtypes = [_vp, _vp, _vp, _vp, _vp, _i, _i, _i, _f, _u64,
-                               _i, _vp]
+                               _i, _i, _vp]
     lib.fei_advance.argtypes = [_vp, _vp, _i, _i, _vp]
     lib.fei_attn_prefill.argtypes = [_vp, _vp, _vp, _vp, _vp, _vp,
                                      _i, _i, _i, _i, _i, _i, _f, _i, _l, _vp]
@@ -67,7 +67,7 @@ def _try_load() -> None:
                                           _vp, _i, _i, _i, _i, _i, _f,
                                           _l, _l, _vp]
     lib.fei_sample_onepass.argtypes = [_vp, _vp, _vp, _vp, _i, _i, _f, _u64,
-                                       _i, _vp]
+                                       _i, _i, _vp]
     lib.fei_sample_shard.argtypes = [_vp, _vp, _vp, _i, _i, _i, _f, _u64, _vp]
     lib.fei_stream_layer_check.argtypes = [_i, _i, _i, _i, _i]
     lib.fei_stream_layer_check.restype = _i
@@ -367,7 +367,7 @@ def sample(logits: torch.Tensor, token: torch.Tensor,
            temperature: float = 0.0, seed: int = 0,
            nchunks: int = 64) -> torch.Tensor:
     """Greedy (T<=0) or Gumbel-max categorical (T>0) sampling.
-    logits [B,V] bf16 -> token [B] int32 (written in place; also appended to
+    logits [B,V] bf16 or float32 -> token [B] int32 (written in place; also appended to
     out_tokens[b, step] when given). All state on device (hipGraph-safe)."""
     B, V = logits.shape
     if not logits.is_cuda:
@@ -388,15 +388,17 @@ def sample(logits: torch.Tensor, token: torch.Tensor,
                     out_tokens[b, st] = t[b]
         return token
     lib = require_lib()
+    f32 = 1 if logits.dtype == torch.float32 else 0
     max_new = out_tokens.shape[1] if out_tokens is not None else 0
     out_ptr = _ptr(out_tokens) if out_tokens is not None else None
     if B <= 8:
         lib.fei_sample_onepass(_ptr(logits), _ptr(token), out_ptr, _ptr(step),
-                               B, V, temperature, seed, max_new, _stream())
+                               B, V, temperature, seed, max_new, f32,
+                               _stream())
     else:
         lib.fei_sample(_ptr(logits), _ptr(token), out_ptr, _ptr(step),
                        _ptr(workspace), B, V, nchunks, temperature, seed,
-                       max_new, _stream())
+                       max_new, f32, _stream())
     return token
 
 

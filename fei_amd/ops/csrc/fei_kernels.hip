@@ -11,6 +11,10 @@
 #include "fei_common.h"
 #include <cstdlib>  // getenv: FEI_ATTN_KV_NT (decode KV cache policy)
 
+// a logit as float: bfloat16 bits or float
+__device__ __forceinline__ float logit(u16 v) { return bf2f(v); }
+__device__ __forceinline__ float logit(float v) { return v; }
+
 extern "C" {
 
 // ---------------------------------------------------------------------------
@@ -755,8 +759,11 @@ void fei_swiglu(void* out, const void* gate_up, long rows, int inter,
 // kernels is hipGraph-replayable.
 // ws: [B, nchunks, 2] f32 (value, idx-as-float-bits via int store).
 // ---------------------------------------------------------------------------
+}  // extern "C"
+
+template <typename T>
 __global__ void __launch_bounds__(256)
-k_sample_partial(const u16* __restrict__ logits, float* __restrict__ ws,
+k_sample_partial(const T* __restrict__ logits, float* __restrict__ ws,
                  int B, int vocab, int nchunks, float temperature,
                  u64 seed, const int* __restrict__ step) {
   const int chunk = blockIdx.x;
@@ -769,7 +776,7 @@ k_sample_partial(const u16* __restrict__ logits, float* __restrict__ ws,
   int besti = start;
   const float invT = temperature > 0.f ? 1.f / temperature : 1.f;
   for (int i = start + threadIdx.x; i < end; i += blockDim.x) {
-    float v = bf2f(logits[(long)b * vocab + i]) * invT;
+    float v = logit(logits[(long)b * vocab + i]) * invT;
     if (temperature > 0.f) {
       float u = hash_uniform(seed ^ (st * 0x51ed27f1ull) ^ ((u64)b << 40) ^ (u64)i);
       v += -__logf(-__logf(u));
@@ -795,6 +802,8 @@ k_sample_partial(const u16* __restrict__ logits, float* __restrict__ ws,
     ((int*)ws)[((long)b * nchunks + chunk) * 2 + 1] = besti;
   }
 }
+
+extern "C" {
 
 __global__ void k_sample_final(const float* __restrict__ ws,
                                int* __restrict__ token,
@@ -827,11 +836,16 @@ __global__ void k_sample_final(const float* __restrict__ ws,
 
 void fei_sample(const void* logits, int* token, int* out_tokens,
                 const int* step, float* ws, int B, int vocab, int nchunks,
-                float temperature, u64 seed, int max_new,
+                float temperature, u64 seed, int max_new, int f32,
                 hipStream_t stream) {
-  hipLaunchKernelGGL(k_sample_partial, dim3(nchunks, B), dim3(256), 0, stream,
-                     (const u16*)logits, ws, B, vocab, nchunks, temperature,
-                     seed, step);
+  if (f32)
+    hipLaunchKernelGGL(k_sample_partial<float>, dim3(nchunks, B), dim3(256), 0,
+                       stream, (const float*)logits, ws, B, vocab, nchunks,
+                       temperature, seed, step);
+  else
+    hipLaunchKernelGGL(k_sample_partial<u16>, dim3(nchunks, B), dim3(256), 0,
+                       stream, (const u16*)logits, ws, B, vocab, nchunks,
+                       temperature, seed, step);
   hipLaunchKernelGGL(k_sample_final, dim3(B), dim3(64), 0, stream,
                      ws, token, out_tokens, step, B, nchunks, max_new);
 }
@@ -861,10 +875,9 @@ void fei_advance(int* pos, int* step, int B, int max_pos,
 // the whole vocab row; replaces the partial+final pair (one node, no
 // workspace round trip).
 // ---------------------------------------------------------------------------
-extern "C" {
-
+template <typename T>
 __global__ void __launch_bounds__(1024)
-k_sample_onepass(const u16* __restrict__ logits, int* __restrict__ token,
+k_sample_onepass(const T* __restrict__ logits, int* __restrict__ token,
                  int* __restrict__ out_tokens, const int* __restrict__ step,
                  int B, int vocab, float temperature, u64 seed, int max_new) {
   const int b = blockIdx.x;
@@ -873,14 +886,17 @@ k_sample_onepass(const u16* __restrict__ logits, int* __restrict__ token,
   const float invT = temperature > 0.f ? 1.f / temperature : 1.f;
   float best = -1.0f / 0.0f;
   int besti = 0x7fffffff;
-  const s16x8* row = (const s16x8*)(logits + (long)b * vocab);
-  const int nv = vocab >> 3;
+  const T* row = logits + (long)b * vocab;
+  // rows of a vocabulary that is no multiple of 8 are not 16-byte aligned
+  const int nv = (vocab & 7) ? 0 : vocab >> 3;
   for (int i = tid; i < nv; i += blockDim.x) {
-    s16x8 v8 = row[i];
+    T v8[8];
+    __builtin_memcpy(v8, __builtin_assume_aligned(row + i * 8, 16),
+                     sizeof(v8));
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
       const int idx = i * 8 + j;
-      float v = bf2f((u16)v8[j]) * invT;
+      float v = logit(v8[j]) * invT;
       if (temperature > 0.f) {
         float u = hash_uniform(seed ^ (st * 0x51ed27f1ull) ^ ((u64)b << 40) ^ (u64)idx);
         v += -__logf(-__logf(u));
@@ -890,7 +906,7 @@ k_sample_onepass(const u16* __restrict__ logits, int* __restrict__ token,
   }
   // tail (vocab % 8)
   for (int idx = nv * 8 + tid; idx < vocab; idx += blockDim.x) {
-    float v = bf2f(logits[(long)b * vocab + idx]) * invT;
+    float v = logit(row[idx]) * invT;
     if (temperature > 0.f) {
       float u = hash_uniform(seed ^ (st * 0x51ed27f1ull) ^ ((u64)b << 40) ^ (u64)idx);
       v += -__logf(-__logf(u));
@@ -920,12 +936,19 @@ k_sample_onepass(const u16* __restrict__ logits, int* __restrict__ token,
   }
 }
 
+extern "C" {
+
 void fei_sample_onepass(const void* logits, int* token, int* out_tokens,
                         const int* step, int B, int vocab, float temperature,
-                        u64 seed, int max_new, hipStream_t stream) {
-  hipLaunchKernelGGL(k_sample_onepass, dim3(B), dim3(1024), 0, stream,
-                     (const u16*)logits, token, out_tokens, step, B, vocab,
-                     temperature, seed, max_new);
+                        u64 seed, int max_new, int f32, hipStream_t stream) {
+  if (f32)
+    hipLaunchKernelGGL(k_sample_onepass<float>, dim3(B), dim3(1024), 0, stream,
+                       (const float*)logits, token, out_tokens, step, B, vocab,
+                       temperature, seed, max_new);
+  else
+    hipLaunchKernelGGL(k_sample_onepass<u16>, dim3(B), dim3(1024), 0, stream,
+                       (const u16*)logits, token, out_tokens, step, B, vocab,
+                       temperature, seed, max_new);
 }
 
 // Shard sampler for tensor-parallel decode: each rank samples over its OWN

@@ -311,7 +311,8 @@ def main(argv=None) -> int:
     p = argparse.ArgumentParser("fei-api",
                                 description="OpenAI-style local serving API")
     p.add_argument("--model", default=None,
-                   help="default: llama3-8b on GPU, llama3-tiny on CPU")
+                   help="registered name, or a folder with config.json and "
+                        "model.safetensors; default: llama3-8b on GPU, llama3-tiny on CPU")
     p.add_argument("--host", default="127.0.0.1")
     p.add_argument("--port", type=int, default=8123)
     p.add_argument("--check", action="store_true",

@@ -167,7 +167,9 @@ def build_parser() -> argparse.ArgumentParser:
                    version=f"fei_amd {__version__}")
     p.add_argument("--provider", choices=["local", "stub", "scripted"],
                    default=None)
-    p.add_argument("--model", default=None)
+    p.add_argument("--model", default=None,
+                   help="registered name (fei models), or a folder with "
+                        "config.json and model.safetensors")
     p.add_argument("--api-key", default=None,
                    help="API key (reference-compatible; unused by local)")
     p.add_argument("--debug", action="store_true", help="debug logging")
@@ -201,6 +203,7 @@ def build_parser() -> argparse.ArgumentParser:
     b = sub.add_parser("serve", help="run the memdir HTTP server")
     b.add_argument("--port", type=int, default=5000)
 
+    sub.add_parser("models", help="list the registered models")
     sub.add_parser("doctor", help="environment and kernel diagnostics")
     return p
 
@@ -315,6 +318,12 @@ def main(argv: Optional[List[str]] = None) -> int:
     if args.cmd == "serve":
         from fei_amd.memdir.run_server import main as serve_main
         return serve_main(["--port", str(args.port)])
+    if args.cmd == "models":
+        from fei_amd.engine.config import MODEL_SPECS
+        for name, spec in sorted(MODEL_SPECS.items()):
+            print(f"{name:14s} {spec.arch:8s} "
+                  f"{spec.params_bytes() / 2e9:7.3f}B parameters")
+        return 0
     if args.cmd == "doctor":
         return run_doctor()
 
