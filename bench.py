@@ -46,8 +46,19 @@ def main() -> int:
                    help="tensor-parallel degree: the W ranks run ONE agent "
                         "sharded over RCCL/xGMI instead of W independent "
                         "agents (requires world_size == tp)")
+    p.add_argument("--compare", default=None, metavar="MODEL,MODEL,...",
+                   help="instead of the benchmark: prefill and decode "
+                        "throughput of these models, one JSON line per model "
+                        "and batch (1 and 8, or --batch)")
     args = p.parse_args()
 
+    if args.compare:
+        from fei_amd.engine.compare_bench import compare
+        gpu = torch.cuda.is_available()
+        compare(args.compare.split(","),
+                [args.batch] if "--batch" in sys.argv else [1, 8],
+                [512, 2048, 4096] if gpu else [32], 64 if gpu else 4)
+        return 0
     if args.stream:
         os.environ["FEI_STREAM_DECODE"] = "1"
     rank = int(os.environ.get("RANK", "0"))

@@ -17,6 +17,7 @@ from __future__ import annotations
 from dataclasses import dataclass, field
 from typing import Dict, List, Optional, Sequence, Tuple
 
+import numpy as np
 import torch
 
 from fei_amd.engine.kv_cache import HybridCache
@@ -45,9 +46,9 @@ class RaggedBatch:
     def n_rows(self) -> int:
         return self.tokens.shape[0]
 
-    def _upload(self, rows: List[List[int]], width: int) -> torch.Tensor:
-        t = torch.tensor(rows, dtype=torch.int32).view(-1, width)
-        return t.to(self.tokens.device)
+    def _upload(self, rows, width: int) -> torch.Tensor:
+        t = torch.from_numpy(np.asarray(rows, dtype=np.int32))
+        return t.view(-1, width).to(self.tokens.device)
 
     def key_plan(self, window: Optional[int]):
         """What the prompt portions read through a window: per portion
@@ -61,12 +62,12 @@ class RaggedBatch:
                 k0 = 0 if window is None else max(0, pos0 - window + 1)
                 spans.append([row, n, pos0, k0, at])
                 n_keys = pos0 + n - k0
-                owner += [p] * n_keys
+                owner.append(np.full(n_keys, p, dtype=np.int32))
                 at += n_keys
                 tiles += [[p, q] for q in range(0, n, Q_TILE)]
             self._plans[key] = (self._upload(spans, 5), at,
                                 self._upload(tiles, 2),
-                                self._upload(owner, 1).view(-1))
+                                self._upload(np.concatenate(owner), 1).view(-1))
         return self._plans[key]
 
     def chunk_plan(self):
@@ -129,10 +130,10 @@ class StepRunner:
     def _tables(self, seqs: Sequence[int]) -> Tuple[torch.Tensor, torch.Tensor]:
         blocks = [self.cache.table(s).blocks for s in seqs]
         W = max(max((len(b) for b in blocks), default=1), 1)
-        table = torch.full((len(seqs), W), self.cache.scratch_block,
-                           dtype=torch.int32)
+        host = np.full((len(seqs), W), self.cache.scratch_block, np.int32)
         for i, b in enumerate(blocks):
-            table[i, :len(b)] = torch.tensor(b, dtype=torch.int32)
+            host[i, :len(b)] = b
+        table = torch.from_numpy(host)
         slots = torch.tensor([self.cache.slot(s) for s in seqs],
                              dtype=torch.int32)
         return table.to(self.device), slots.to(self.device)
@@ -152,7 +153,8 @@ class StepRunner:
         for e in entries:
             if not len(e.tokens):
                 raise ValueError("an entry needs at least one token")
-            if min(e.tokens) < 0 or max(e.tokens) >= V:
+            t = np.asarray(e.tokens)
+            if t.min() < 0 or t.max() >= V:
                 raise ValueError(f"token outside the vocabulary of {V}")
             if any(w < 0 or w >= len(e.tokens) for w in e.want):
                 raise ValueError("a wanted place is outside the entry")
@@ -163,30 +165,29 @@ class StepRunner:
                                        self.length[e.seq] + len(e.tokens))
         order = sorted(range(len(entries)),
                        key=lambda i: len(entries[i].tokens) > 1)
-        tokens: List[int] = []
-        pos: List[int] = []
-        row_seq: List[int] = []
+        # token, position and sequence of every row
+        meta = np.empty((3, sum(len(e.tokens) for e in entries)), np.int32)
         portions: List[Tuple[int, int, int]] = []
         first_row: Dict[int, int] = {}
-        n_dec = 0
+        n_dec = row = 0
         for s, i in enumerate(order):
             e = entries[i]
             p0, n = self.length[e.seq], len(e.tokens)
-            first_row[i] = len(tokens)
+            first_row[i] = row
             if n == 1:
                 n_dec += 1
             else:
-                portions.append((len(tokens), n, p0))
-            tokens += [int(t) for t in e.tokens]
-            pos += range(p0, p0 + n)
-            row_seq += [s] * n
+                portions.append((row, n, p0))
+            meta[0, row:row + n] = e.tokens
+            meta[1, row:row + n] = np.arange(p0, p0 + n)
+            meta[2, row:row + n] = s
+            row += n
         table, slots = self._tables([entries[i].seq for i in order])
         want = [first_row[i] + w for i, e in enumerate(entries)
                 for w in e.want]
-        meta = torch.tensor([tokens, pos, row_seq],
-                            dtype=torch.int32).to(self.device)
+        rows = torch.from_numpy(meta).to(self.device)
         return RaggedBatch(
-            tokens=meta[0].long(), pos=meta[1], row_seq=meta[2], table=table,
+            tokens=rows[0].long(), pos=rows[1], row_seq=rows[2], table=table,
             slots=slots, n_dec=n_dec, portions=portions,
             want_rows=None if all_rows else torch.tensor(
                 want, dtype=torch.int64, device=self.device))

@@ -125,7 +125,8 @@ def build_if_missing() -> None:
 
 
 def _stream() -> int:
-    return torch.cuda.current_stream().cuda_stream
+    # the raw handle: a Stream object per launch costs more than the launch
+    return torch._C._cuda_getCurrentRawStream(torch.cuda.current_device())
 
 
 def _ptr(t: torch.Tensor) -> int:

@@ -439,7 +439,7 @@ void fei_gemv_swiglu_norm(void* out, const void* res, const void* wn,
 // k_gemv<8> (profiles/r02_batch_attention.md); this MFMA tile beats it
 // on every llama shape (qkv 1.45x, o 1.43x, down 1.27x, stacked gate/up
 // 1.65x — experimental/gemv_mfma.hip, numerics exact vs the VALU form).
-// Structure: 16 n-rows per workgroup, each wave owns a K-QUARTER with
+// Structure: 16 n-rows per workgroup, each of NW waves owns K/NW with
 // wave-private double-buffered LDS staging (register prefetch overlaps
 // the next tile's loads with the current tile's MFMAs; same-wave ds
 // ordering needs no barriers), one end-of-kernel cross-wave C reduce.
@@ -454,8 +454,8 @@ namespace {
 
 typedef __attribute__((ext_vector_type(4))) float f32x4_g;
 
-template <bool NTW, int EPI>
-__global__ void __launch_bounds__(256)
+template <bool NTW, int EPI, int NW = 4>
+__global__ void __launch_bounds__(NW * 64)
 k_gemm_m8(void* __restrict__ outp, const u16* __restrict__ x,
           const u16* __restrict__ w, int M, int N, int K, Epilogue ep) {
   const int n0 = blockIdx.x * GEMM_NT;
@@ -463,11 +463,11 @@ k_gemm_m8(void* __restrict__ outp, const u16* __restrict__ x,
   const int wv = tid >> 6;
   const int lane = tid & 63;
   const int l15 = lane & 15, lg = lane >> 4;
-  __shared__ u16 wt[4][2][GEMM_NT * GEMM_KC];
-  __shared__ float cred[4][16][16];
+  __shared__ u16 wt[NW][2][GEMM_NT * GEMM_KC];
+  __shared__ float cred[NW][16][16];
 
   f32x4_g acc = {0.f, 0.f, 0.f, 0.f};
-  const int kq = K / 4;
+  const int kq = K / NW;
   const int nv8 = GEMM_KC / 8;
   const int k_lo = wv * kq, k_hi = (wv + 1) * kq;
   const int arow = l15 < M ? l15 : M - 1;
@@ -510,8 +510,9 @@ k_gemm_m8(void* __restrict__ outp, const u16* __restrict__ x,
   if (wv == 0) {
     for (int i = lane; i < M * 16; i += 64) {
       const int m = i / 16, n = i % 16;
-      const float v = cred[0][m][n] + cred[1][m][n] + cred[2][m][n] +
-                      cred[3][m][n];
+      float v = cred[0][m][n] + cred[1][m][n] + cred[2][m][n] + cred[3][m][n];
+#pragma unroll
+      for (int c = 4; c < NW; ++c) v += cred[c][m][n];
       epilogue<EPI>(outp, (long)m * N + n0 + n, n0 + n, v, ep);
     }
   }
@@ -520,19 +521,26 @@ k_gemm_m8(void* __restrict__ outp, const u16* __restrict__ x,
 }  // namespace
 
 // float32 results: residual != 0 adds to out, otherwise out is
-// softcap(acc * scale, cap) + bias (cap 0: none; bias may be null).
+// softcap(acc * scale, cap) + bias (cap 0: none; bias may be null). With few
+// columns more waves share out K, so that the weight stream fills the chip.
 extern "C" void fei_gemm_m8_f32(void* out, const void* x, const void* w,
                                 const float* bias, int M, int N, int K,
                                 int residual, float scale, float cap,
                                 hipStream_t stream) {
   dim3 grid(N / GEMM_NT);
   const Epilogue ep{bias, scale, cap};
-  if (residual)
-    hipLaunchKernelGGL((k_gemm_m8<false, EPI_RES>), grid, dim3(256), 0, stream,
-                       out, (const u16*)x, (const u16*)w, M, N, K, ep);
-  else
-    hipLaunchKernelGGL((k_gemm_m8<false, EPI_F32>), grid, dim3(256), 0, stream,
-                       out, (const u16*)x, (const u16*)w, M, N, K, ep);
+#define M8(EPI, NW)                                                         \
+  hipLaunchKernelGGL((k_gemm_m8<false, EPI, NW>), grid, dim3(NW * 64), 0,   \
+                     stream, out, (const u16*)x, (const u16*)w, M, N, K, ep)
+#define BY_NW(EPI)                                                          \
+  do {                                                                      \
+    if (N <= 4096 && K % 2048 == 0) M8(EPI, 16);                            \
+    else if (N <= 8192) M8(EPI, 8);                                         \
+    else M8(EPI, 4);                                                        \
+  } while (0)
+  if (residual) BY_NW(EPI_RES); else BY_NW(EPI_F32);
+#undef BY_NW
+#undef M8
 }
 
 extern "C" void fei_gemm_m8(void* out, const void* x, const void* w, int M,

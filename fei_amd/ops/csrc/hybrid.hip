@@ -112,16 +112,18 @@ k_softcap(float* __restrict__ y, long n, float scale, float cap) {
     y[i] = softcap(y[i], scale, cap);
 }
 
-// Two weight rows per wave, streamed 16 bytes a lane; x comes from L1/L2.
+// Two weight rows, streamed 16 bytes a lane by the lanes of ``step`` / 64
+// waves; the sums are this wave's. x comes from L1/L2.
 template <int M, bool NT>
 __device__ __forceinline__ void two_rows(const u16* __restrict__ x,
                                          const u16* __restrict__ w0,
                                          const u16* __restrict__ w1, int K,
-                                         int lane, float* a0, float* a1) {
+                                         int first, int step, float* a0,
+                                         float* a1) {
 #pragma unroll
   for (int m = 0; m < M; ++m) a0[m] = a1[m] = 0.f;
   const int nv = K >> 3;
-  for (int i = lane; i < nv; i += 64) {
+  for (int i = first; i < nv; i += step) {
     const s16x8 v0 = NT ? __builtin_nontemporal_load((const s16x8*)w0 + i)
                         : ((const s16x8*)w0)[i];
     const s16x8 v1 = NT ? __builtin_nontemporal_load((const s16x8*)w1 + i)
@@ -155,7 +157,8 @@ k_gemv_mix_in(u16* __restrict__ proj, u16* __restrict__ act,
   float a0[M], a1[M];
   if (u < units) {
     const int r0 = 2 * u, r1 = min(2 * u + 1, n_mix - 1);
-    two_rows<M, NT>(x1, w + (long)r0 * K, w + (long)r1 * K, K, lane, a0, a1);
+    two_rows<M, NT>(x1, w + (long)r0 * K, w + (long)r1 * K, K, lane, 64, a0,
+                    a1);
     if (lane == 0) {
 #pragma unroll
       for (int m = 0; m < M; ++m) {
@@ -166,7 +169,7 @@ k_gemv_mix_in(u16* __restrict__ proj, u16* __restrict__ act,
   } else if (u - units < ff) {
     const int i = u - units;
     two_rows<M, NT>(x2, w + (long)(n_mix + i) * K,
-                    w + (long)(n_mix + ff + i) * K, K, lane, a0, a1);
+                    w + (long)(n_mix + ff + i) * K, K, lane, 64, a0, a1);
     if (lane == 0) {
 #pragma unroll
       for (int m = 0; m < M; ++m) {
@@ -177,17 +180,37 @@ k_gemv_mix_in(u16* __restrict__ proj, u16* __restrict__ act,
   }
 }
 
-template <int M, bool NT, int EPI>
+// out rows by an epilogue, two weight rows at a time. KSPLIT 1: a wave takes
+// two whole rows. KSPLIT 4: the block's waves share two rows, for products
+// with too few rows to fill the chip.
+template <int M, bool NT, int EPI, int KSPLIT>
 __global__ void __launch_bounds__(256)
 k_gemv_f32(float* __restrict__ out, const u16* __restrict__ x,
            const u16* __restrict__ w, int N, int K, Epilogue ep) {
-  const int lane = threadIdx.x & 63;
-  const int n0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * 2;
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int n0 = (KSPLIT == 1 ? blockIdx.x * 4 + wid : blockIdx.x) * 2;
   if (n0 >= N) return;
   const int n1 = min(n0 + 1, N - 1);
   float a0[M], a1[M];
-  two_rows<M, NT>(x, w + (long)n0 * K, w + (long)n1 * K, K, lane, a0, a1);
-  if (lane == 0) {
+  two_rows<M, NT>(x, w + (long)n0 * K, w + (long)n1 * K, K,
+                  KSPLIT == 1 ? lane : wid * 64 + lane, KSPLIT * 64, a0, a1);
+  if (KSPLIT > 1) {
+    __shared__ float red[4][2][M];
+    if (lane == 0) {
+#pragma unroll
+      for (int m = 0; m < M; ++m) {
+        red[wid][0][m] = a0[m];
+        red[wid][1][m] = a1[m];
+      }
+    }
+    __syncthreads();
+    if (threadIdx.x >= 2 * M) return;
+    const int m = threadIdx.x >> 1, n = threadIdx.x & 1;
+    if (n == 1 && n1 == n0) return;
+    epilogue<EPI>(out, (long)m * N + n0 + n, n0 + n,
+                  (red[0][n][m] + red[1][n][m]) + (red[2][n][m] + red[3][n][m]),
+                  ep);
+  } else if (lane == 0) {
 #pragma unroll
     for (int m = 0; m < M; ++m) {
       epilogue<EPI>(out, (long)m * N + n0, n0, a0[m], ep);
@@ -278,20 +301,26 @@ void fei_gemv_mix_in(void* proj, void* act, const void* x1, const void* x2,
 void fei_gemv_f32(void* out, const void* x, const void* w, const float* bias,
                   int M, int N, int K, int residual, float scale, float cap,
                   int nt, hipStream_t stream) {
-  const dim3 grid((N + 7) / 8);
+  const bool share = N < 8192;             // rows alone do not fill the chip
+  const dim3 grid(share ? (N + 1) / 2 : (N + 7) / 8);
   const Epilogue ep{bias, scale, cap};
-#define LAUNCH(MV, NTV, EPI)                                                \
-  hipLaunchKernelGGL((k_gemv_f32<MV, NTV, EPI>), grid, dim3(256), 0,        \
+#define LAUNCH(MV, NTV, EPI, KSP)                                           \
+  hipLaunchKernelGGL((k_gemv_f32<MV, NTV, EPI, KSP>), grid, dim3(256), 0,   \
                      stream, (float*)out, (const u16*)x, (const u16*)w, N,  \
                      K, ep)
+#define BY_NT(MV, EPI, KSP)                                                 \
+  do {                                                                      \
+    if (nt) LAUNCH(MV, true, EPI, KSP); else LAUNCH(MV, false, EPI, KSP);   \
+  } while (0)
 #define CALL(MV)                                                            \
   if (residual) {                                                           \
-    if (nt) LAUNCH(MV, true, EPI_RES); else LAUNCH(MV, false, EPI_RES);     \
+    if (share) BY_NT(MV, EPI_RES, 4); else BY_NT(MV, EPI_RES, 1);           \
   } else {                                                                  \
-    if (nt) LAUNCH(MV, true, EPI_F32); else LAUNCH(MV, false, EPI_F32);     \
+    if (share) BY_NT(MV, EPI_F32, 4); else BY_NT(MV, EPI_F32, 1);           \
   }
   BY_M(M, CALL)
 #undef CALL
+#undef BY_NT
 #undef LAUNCH
 }
 

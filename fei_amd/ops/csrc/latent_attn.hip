@@ -177,7 +177,9 @@ __device__ __forceinline__ T part_of(float v, int i) {
 
 // Decode partials. grid (splits, ceil(heads / 16), B), 4 waves. The visible
 // keys of row b are cut into ``splits`` chunks of a multiple of KT keys; a
-// block walks its chunk in tiles of KT cached rows held in LDS.
+// block walks its chunk in tiles of KT cached rows held in LDS. For the scores
+// the waves share out the 32-wide steps along a row (their sums meet in LDS),
+// for the weighted sum the columns.
 // NCT: 16-column tiles of the latent per wave (kr <= 64 * NCT).
 // part_o [B, H, splits, kr] unnormalised, part_ml [B, H, splits, 2].
 template <typename T, int NCT>
@@ -189,15 +191,16 @@ k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
                 int vec) {
   typedef typename El<T>::frag frag;
   constexpr int NP = Parts<T>::n;
+  constexpr int NQ = 9;                    // steps per wave: R <= 4 * 9 * 32
+  constexpr int NL = 6;                    // row loads in flight per thread
   extern __shared__ __align__(16) char smem[];
   const int R = g.kr + g.rot;
   const int KP = (KT + 31) / 32 * 32;      // P columns, zero beyond KT
   const int KPs = KP + 8;
-  T* qs = (T*)smem;                        // [16][Rs]
-  T* ks = qs + 16 * Rs;                    // [KP][Rs]
+  T* ks = (T*)smem;                        // [KP][Rs]
   T* ph = ks + KP * Rs;                    // [NP][16][KPs]
-  float* ss = (float*)(ph + NP * 16 * KPs);  // [16][KT + 1]
-  float* al = ss + 16 * (KT + 1);          // [16]
+  float* ss = (float*)(ph + NP * 16 * KPs);  // [4][16][KT + 1]
+  float* al = ss + 64 * (KT + 1);          // [16]
 
   const int split = blockIdx.x, h0 = blockIdx.y * 16, b = blockIdx.z;
   const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63;
@@ -218,11 +221,27 @@ k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
     return;
   }
 
-  // queries, zero beyond the heads and beyond R; P and the tail rows zero
-  for (int i = tid; i < 16 * Rs; i += 256) {
-    const int h = i / Rs, c = i - h * Rs;
-    qs[i] = (h < nh && c < R) ? qa[((long)b * g.heads + h0 + h) * R + c]
-                              : El<T>::st(0.f);
+  // queries of this wave's steps, zero beyond the heads and beyond R
+  const int ksteps = (R + 31) / 32;
+  frag q[NQ];
+  {
+    const T* qr = qa + ((long)b * g.heads + h0 + min(l15, nh - 1)) * R;
+#pragma unroll
+    for (int i = 0; i < NQ; ++i) {
+      const int k = w + 4 * i;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) q[i][j] = 0;
+      if (k < ksteps && l15 < nh) {
+        const int c = k * 32 + 8 * lg;
+        if (vec) {
+          if (c < R) q[i] = ld8(qr + c);
+        } else {
+#pragma unroll
+          for (int j = 0; j < 8; ++j)
+            if (c + j < R) q[i][j] = qr[c + j];
+        }
+      }
+    }
   }
   for (int i = tid; i < NP * 16 * KPs; i += 256) ph[i] = El<T>::st(0.f);
   for (int i = KT * Rs + tid; i < KP * Rs; i += 256) ks[i] = El<T>::st(0.f);
@@ -232,20 +251,29 @@ k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
   for (int i = 0; i < NCT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
   // row 4w + lg of the scores is this 16-lane group's
   float m = NEG_INF, l = 0.f;
-  const int ksteps = (R + 31) / 32;
 
   for (int t0 = lo; t0 < hi; t0 += KT) {
     __syncthreads();
     if (vec) {
       const int nv = Rs / 8 - 1;           // vec8 slots that may be read
-      for (int i = tid; i < KT * nv; i += 256) {
-        const int r = i / nv, c = (i - r * nv) * 8;
-        frag v;
+      for (int i0 = tid; i0 < KT * nv; i0 += 256 * NL) {
+        frag v[NL];
 #pragma unroll
-        for (int j = 0; j < 8; ++j) v[j] = 0;
-        if (t0 + r < hi && c < R)
-          v = ld8(rows + cache_row(table, W, b, k0 + t0 + r, bs_log) * R + c);
-        st8(ks + r * Rs + c, v);
+        for (int u = 0; u < NL; ++u) {
+          const int i = i0 + u * 256;
+          const int r = i / nv, c = (i - r * nv) * 8;
+#pragma unroll
+          for (int j = 0; j < 8; ++j) v[u][j] = 0;
+          if (i < KT * nv && t0 + r < hi && c < R)
+            v[u] = ld8(rows +
+                       cache_row(table, W, b, k0 + t0 + r, bs_log) * R + c);
+        }
+#pragma unroll
+        for (int u = 0; u < NL; ++u) {
+          const int i = i0 + u * 256;
+          const int r = i / nv, c = (i - r * nv) * 8;
+          if (i < KT * nv) st8(ks + r * Rs + c, v[u]);
+        }
       }
     } else {
       for (int i = tid; i < KT * Rs; i += 256) {
@@ -256,31 +284,47 @@ k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
       }
     }
     __syncthreads();
-    for (int kt = w; kt < KT / 16; kt += 4) {
+    for (int kt = 0; kt < KT / 16; ++kt) {
       f32x4 s = {0.f, 0.f, 0.f, 0.f};
-      for (int k = 0; k < ksteps; ++k)
-        s = mma(ld8(qs + l15 * Rs + k * 32 + 8 * lg),
-                ld8(ks + (kt * 16 + l15) * Rs + k * 32 + 8 * lg), s);
+#pragma unroll
+      for (int i = 0; i < NQ; ++i)
+        if (w + 4 * i < ksteps)
+          s = mma(q[i], ld8(ks + (kt * 16 + l15) * Rs + (w + 4 * i) * 32 +
+                            8 * lg), s);
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        ss[(4 * lg + r) * (KT + 1) + kt * 16 + l15] =
-            t0 + kt * 16 + l15 < hi ? s[r] * g.scale : NEG_INF;
+        ss[(w * 16 + 4 * lg + r) * (KT + 1) + kt * 16 + l15] = s[r];
     }
     __syncthreads();
     {
       const int row = 4 * w + lg;
+      float sv[4];
       float mx = m;
-      for (int c = l15; c < KT; c += 16) mx = fmaxf(mx, ss[row * (KT + 1) + c]);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int c = l15 + 16 * i;
+        sv[i] = NEG_INF;
+        if (c < KT && t0 + c < hi) {
+          const float* x = ss + row * (KT + 1) + c;
+          const int st = 16 * (KT + 1);
+          sv[i] = ((x[0] + x[st]) + (x[2 * st] + x[3 * st])) * g.scale;
+        }
+        mx = fmaxf(mx, sv[i]);
+      }
 #pragma unroll
       for (int off = 1; off < 16; off <<= 1) mx = fmaxf(mx, __shfl_xor(mx, off));
       const float a = El<T>::ex(m - mx);   // a tile has a visible key: mx is finite
       float sum = 0.f;
-      for (int c = l15; c < KT; c += 16) {
-        const float e = El<T>::ex(ss[row * (KT + 1) + c] - mx);
-        sum += e;
 #pragma unroll
-        for (int i = 0; i < NP; ++i)
-          ph[(i * 16 + row) * KPs + c] = part_of<T>(e, i);
+      for (int i = 0; i < 4; ++i) {
+        const int c = l15 + 16 * i;
+        if (c < KT) {
+          const float e = El<T>::ex(sv[i] - mx);
+          sum += e;
+#pragma unroll
+          for (int pi = 0; pi < NP; ++pi)
+            ph[(pi * 16 + row) * KPs + c] = part_of<T>(e, pi);
+        }
       }
 #pragma unroll
       for (int off = 1; off < 16; off <<= 1) sum += __shfl_xor(sum, off);
@@ -332,16 +376,27 @@ k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
 }
 
 // Combine the partials of one head, apply W_uv and the gate. grid (heads,
-// ceil(vdim / 64), B); a wave takes 16 value rows.
+// ceil(vdim / 16), B); a wave takes 4 value rows, whose first weights it reads
+// ahead of the combination.
 template <typename T, bool VEC>
 __global__ void __launch_bounds__(256)
 k_latent_out(T* __restrict__ out, long os, const float* __restrict__ part_o,
              const float* __restrict__ part_ml, const T* __restrict__ wuv,
              const T* __restrict__ gate, long gs, Geo g, int splits) {
   __shared__ float wt[64];
-  __shared__ float o[1024];
+  __shared__ __align__(16) float o[1024];
   const int h = blockIdx.x, b = blockIdx.z, tid = threadIdx.x;
+  const int w = tid >> 6, lane = tid & 63;
   const long bh = (long)b * g.heads + h;
+  const int v0 = blockIdx.y * 16 + w * 4;
+  const T* wr = wuv + ((long)h * g.vdim + v0) * g.kr;
+  typename El<T>::frag pre[4];
+  if (VEC) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (v0 + i < g.vdim && lane * 8 < g.kr)
+        pre[i] = ld8(wr + (long)i * g.kr + lane * 8);
+  }
   if (tid < 64) {
     const bool on = tid < splits;
     const float m = on ? part_ml[(bh * splits + tid) * 2] : NEG_INF;
@@ -353,34 +408,45 @@ k_latent_out(T* __restrict__ out, long os, const float* __restrict__ part_o,
   }
   __syncthreads();
   for (int c = tid; c < g.kr; c += 256) {
+    const float* po = part_o + bh * splits * g.kr + c;
     float v = 0.f;
-    for (int s = 0; s < splits; ++s)
-      if (wt[s] > 0.f) v = fmaf(wt[s], part_o[(bh * splits + s) * g.kr + c], v);
+    int s = 0;
+    for (; s + 8 <= splits; s += 8) {
+      float x[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) x[u] = po[(long)(s + u) * g.kr];
+#pragma unroll
+      for (int u = 0; u < 8; ++u)          // an empty split wrote nothing
+        v = wt[s + u] > 0.f ? fmaf(wt[s + u], x[u], v) : v;
+    }
+    for (; s < splits; ++s)
+      v = wt[s] > 0.f ? fmaf(wt[s], po[(long)s * g.kr], v) : v;
     o[c] = v;
   }
   __syncthreads();
-  const int w = tid >> 6, lane = tid & 63;
-#pragma unroll 4
-  for (int i = 0; i < 16; ++i) {
-    const int v = blockIdx.y * 64 + i * 4 + w;
-    if (v >= g.vdim) break;
-    const T* wr = wuv + ((long)h * g.vdim + v) * g.kr;
-    float acc = 0.f;
+  float acc[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    if (v0 + i >= g.vdim) continue;
+    const T* r = wr + (long)i * g.kr;
     if (VEC) {
       for (int c = lane * 8; c < g.kr; c += 512) {
-        const auto wv = ld8(wr + c);
+        const auto wv = c == lane * 8 ? pre[i] : ld8(r + c);
 #pragma unroll
-        for (int j = 0; j < 8; ++j) acc = fmaf(o[c + j], get8(wv, j), acc);
+        for (int j = 0; j < 8; ++j) acc[i] = fmaf(o[c + j], get8(wv, j), acc[i]);
       }
     } else {
       for (int c = lane; c < g.kr; c += 64)
-        acc = fmaf(o[c], El<T>::ld(wr[c]), acc);
+        acc[i] = fmaf(o[c], El<T>::ld(r[c]), acc[i]);
     }
-    acc = wave_reduce_sum(acc);
-    if (lane == 0) {
-      const int col = h * g.vdim + v;
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const float v = wave_reduce_sum(acc[i]);
+    if (lane == 0 && v0 + i < g.vdim) {
+      const int col = h * g.vdim + v0 + i;
       out[(long)b * os + col] = El<T>::st(
-          acc * sigmoid_f(El<T>::ld(gate[(long)b * gs + col])));
+          v * sigmoid_f(El<T>::ld(gate[(long)b * gs + col])));
     }
   }
 }
@@ -412,15 +478,23 @@ k_latent_gather(T* __restrict__ c, T* __restrict__ kr_out,
   }
 }
 
+// Place of (column, key) in the transposed value tile: 64 keys a column in
+// blocks of 8, the block index permuted by the column so that neither the
+// stores (lanes along columns) nor the reads (16 columns, one block) pile up
+// on a bank.
+__device__ __forceinline__ int vt_at(int col, int key) {
+  return col * 64 + ((((key >> 3) ^ col ^ (col >> 3)) & 7) << 3) + (key & 7);
+}
+
 // Flash attention of prompt portions over expanded keys and values.
-// grid (query tiles, heads), 4 waves; a wave owns MR tiles of 16 query rows,
+// grid (heads, query tiles), 4 waves; a wave owns MR tiles of 16 query rows,
 // the block 64*MR of them, in tiles of 64 keys held in LDS: keys row-major,
 // values transposed. tiles [.][2]: portion, first row in it (a tile of the
 // plan is 128 rows; with MR = 1 two blocks share it, blockIdx.z).
 // KS = ceil((dim + rot) / 32), DC = ceil(vdim / 16), rounded up to what is
 // instantiated; zero padding in LDS makes the padded products vanish.
 template <typename T, int KS, int DC, int MR>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, 2)
 k_window_prefill(T* __restrict__ out, long os, const T* __restrict__ proj,
                  long ps, const T* __restrict__ kv, const T* __restrict__ krot,
                  const int* __restrict__ spans, const int* __restrict__ tiles,
@@ -428,16 +502,18 @@ k_window_prefill(T* __restrict__ out, long os, const T* __restrict__ proj,
   typedef typename El<T>::frag frag;
   constexpr int NP = Parts<T>::n;
   constexpr int DS = KS * 32 + 8;          // odd count of 16-byte slots
-  constexpr int VS = 64 + 8;
+  constexpr int PS = 64 + 8;
   extern __shared__ __align__(16) char smem[];
   T* kt = (T*)smem;                        // [64][DS]
-  T* vt = kt + 64 * DS;                    // [DC * 16][VS]
-  T* pl = vt + DC * 16 * VS;               // [4 waves][NP][16][VS]
+  T* vt = kt + 64 * DS;                    // [DC * 16][64], see vt_at
+  T* pl = vt + DC * 16 * 64;               // [4 waves][NP][16][PS]
 
-  const int h = blockIdx.y;
-  const int* sp = spans + tiles[blockIdx.x * 2] * 5;
+  // heads run fastest, so that with 8 | heads a head stays on one XCD and
+  // neighbouring tiles find their common keys in its L2
+  const int h = blockIdx.x;
+  const int* sp = spans + tiles[blockIdx.y * 2] * 5;
   const int row0 = sp[0], cnt = sp[1], pos0 = sp[2], key0 = sp[3], at0 = sp[4];
-  const int q0 = tiles[blockIdx.x * 2 + 1] + (MR == 1 ? blockIdx.z * 64 : 0);
+  const int q0 = tiles[blockIdx.y * 2 + 1] + (MR == 1 ? blockIdx.z * 64 : 0);
   if (q0 >= cnt) return;
   const int qn = min(64 * MR, cnt - q0);
   const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63;
@@ -478,7 +554,7 @@ k_window_prefill(T* __restrict__ out, long os, const T* __restrict__ proj,
   // positions of this tile's queries and of the keys any of them sees
   const int qa = pos0 + q0, qb = qa + qn - 1;
   const int klo = max(first_key(qa, g.window), key0) & ~63;
-  T* pw = pl + w * NP * 16 * VS;
+  T* pw = pl + w * NP * 16 * PS;
 
   for (int t0 = klo; t0 <= qb; t0 += 64) {
     __syncthreads();
@@ -501,7 +577,7 @@ k_window_prefill(T* __restrict__ out, long os, const T* __restrict__ proj,
       // values, two keys at a time so that a transposed store is a pair
       constexpr int NW = DC * 2;
       for (int i = tid; i < 32 * NW; i += 256) {
-        const int r = (i & 31) * 2, c = (i >> 5) * 8;
+        const int r = i / NW * 2, c = i % NW * 8;
         frag a, bb;
 #pragma unroll
         for (int j = 0; j < 8; ++j) { a[j] = 0; bb[j] = 0; }
@@ -514,7 +590,7 @@ k_window_prefill(T* __restrict__ out, long os, const T* __restrict__ proj,
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
           T two[2] = {(T)a[j], (T)bb[j]};
-          __builtin_memcpy(vt + (c + j) * VS + r, two, sizeof(two));
+          __builtin_memcpy(vt + vt_at(c + j, r), two, sizeof(two));
         }
       }
     } else {
@@ -536,7 +612,7 @@ k_window_prefill(T* __restrict__ out, long os, const T* __restrict__ proj,
         if (key >= key0 && key <= qb && c < g.vdim)
           v = kv[(long)(at0 + key - key0) * kvs + (long)g.heads * g.dim +
                  (long)h * g.vdim + c];
-        vt[c * VS + r] = v;
+        vt[vt_at(c, r)] = v;
       }
     }
     __syncthreads();
@@ -588,7 +664,7 @@ k_window_prefill(T* __restrict__ out, long os, const T* __restrict__ proj,
           sum += e;
 #pragma unroll
           for (int pi = 0; pi < NP; ++pi)
-            pw[(pi * 16 + 4 * lg + r) * VS + c * 16 + l15] = part_of<T>(e, pi);
+            pw[(pi * 16 + 4 * lg + r) * PS + c * 16 + l15] = part_of<T>(e, pi);
         }
 #pragma unroll
         for (int off = 1; off < 16; off <<= 1) sum += __shfl_xor(sum, off);
@@ -601,7 +677,7 @@ k_window_prefill(T* __restrict__ out, long os, const T* __restrict__ proj,
       for (int pi = 0; pi < NP; ++pi)
 #pragma unroll
         for (int k = 0; k < 2; ++k)
-          ap[pi][k] = ld8(pw + (pi * 16 + l15) * VS + k * 32 + 8 * lg);
+          ap[pi][k] = ld8(pw + (pi * 16 + l15) * PS + k * 32 + 8 * lg);
       __builtin_amdgcn_wave_barrier();
 #pragma unroll
       for (int d = 0; d < DC; ++d) {
@@ -609,7 +685,7 @@ k_window_prefill(T* __restrict__ out, long os, const T* __restrict__ proj,
         for (int r = 0; r < 4; ++r) o[i][d][r] *= al[r];
 #pragma unroll
         for (int k = 0; k < 2; ++k) {
-          const frag bv = ld8(vt + (d * 16 + l15) * VS + k * 32 + 8 * lg);
+          const frag bv = ld8(vt + vt_at(d * 16 + l15, k * 32 + 8 * lg));
 #pragma unroll
           for (int pi = 0; pi < NP; ++pi)
             o[i][d] = mma(ap[pi][k], bv, o[i][d]);
@@ -642,7 +718,7 @@ int run_decode(T* out, long os, const T* proj, long ps, const T* wuk,
                const T* wuv, const float* nw, const float* rotab, T* rows,
                const int* pos, const int* table, T* qa, float* part_o,
                float* part_ml, int B, int W, int bs_log, Geo g, float eps,
-               int splits, hipStream_t stream) {
+               int splits, int tile, hipStream_t stream) {
   const int R = g.kr + g.rot;
   const bool vkr = g.kr % 8 == 0;
   const dim3 ga(g.heads + 1, (g.kr + 127) / 128, B);
@@ -658,13 +734,12 @@ int run_decode(T* out, long os, const T* proj, long ps, const T* wuk,
   const int Rs = (R + 31) / 32 * 32 + 8;
   auto lds = [&](int KT) {
     const int KP = (KT + 31) / 32 * 32;
-    return (size_t)sizeof(T) * (16 * Rs + KP * Rs +
-                                Parts<T>::n * 16 * (KP + 8)) +
-           4 * (16 * (KT + 1) + 16);
+    return (size_t)sizeof(T) * (KP * Rs + Parts<T>::n * 16 * (KP + 8)) +
+           4 * (64 * (KT + 1) + 16);
   };
-  int KT = 64;
+  int KT = tile;
   while (KT > 16 && lds(KT) > 160 * 1024) KT >>= 1;
-  if (lds(KT) > 160 * 1024) return 1;
+  if (lds(KT) > 160 * 1024 || R > 1152) return 1;
   const dim3 gd(splits, (g.heads + 15) / 16, B);
 #define DEC(N)                                                               \
   do {                                                                       \
@@ -686,7 +761,7 @@ int run_decode(T* out, long os, const T* proj, long ps, const T* wuk,
   else DEC(16);
 #undef DEC
 
-  const dim3 go(g.heads, (g.vdim + 63) / 64, B);
+  const dim3 go(g.heads, (g.vdim + 15) / 16, B);
   const T* gate = proj + (long)g.heads * (g.dim + g.rot) + R;
   if (vkr)
     hipLaunchKernelGGL((k_latent_out<T, true>), go, dim3(256), 0, stream, out,
@@ -702,7 +777,7 @@ void launch_window(T* out, long os, const T* proj, long ps, const T* kv,
                    const T* krot, const int* spans, const int* tiles,
                    int n_tiles, Geo g, int vec, hipStream_t stream) {
   constexpr int MR = sizeof(T) == 2 && KS * 4 + DC * 4 <= 64 ? 2 : 1;
-  const size_t lds = sizeof(T) * (64 * (KS * 32 + 8) + DC * 16 * 72 +
+  const size_t lds = sizeof(T) * (64 * (KS * 32 + 8) + DC * 16 * 64 +
                                   4 * Parts<T>::n * 16 * 72);
   static bool set = false;
   if (!set) {
@@ -711,7 +786,7 @@ void launch_window(T* out, long os, const T* proj, long ps, const T* kv,
                               160 * 1024);
     set = true;
   }
-  const dim3 grid(n_tiles, g.heads, MR == 1 ? 2 : 1);
+  const dim3 grid(g.heads, n_tiles, MR == 1 ? 2 : 1);
   const int gate_off = g.heads * (g.dim + g.rot) + g.kr + g.rot;
   hipLaunchKernelGGL((k_window_prefill<T, KS, DC, MR>), grid, dim3(256), lds,
                      stream, out, os, proj, ps, kv, krot, spans, tiles,
@@ -746,6 +821,7 @@ void run_window(T* out, long os, const T* proj, long ps, const T* kv,
 
 extern "C" {
 
+// tile: keys per LDS tile, 16, 32 or 64; fewer are taken if they do not fit.
 // Returns 0, or 1 if the sizes do not fit the kernel's LDS tiles.
 int fei_latent_decode(void* out, long os, const void* proj, long ps,
                       const void* wuk, const void* wuv, const float* nw,
@@ -753,18 +829,18 @@ int fei_latent_decode(void* out, long os, const void* proj, long ps,
                       const int* table, void* qa, float* part_o,
                       float* part_ml, int B, int W, int bs_log, int heads,
                       int dim, int rot, int vdim, int kr, float scale,
-                      int window, float eps, int splits, int f32,
+                      int window, float eps, int splits, int tile, int f32,
                       hipStream_t stream) {
   const Geo g{heads, dim, rot, vdim, kr, scale, window};
   if (f32)
     return run_decode<float>((float*)out, os, (const float*)proj, ps,
                              (const float*)wuk, (const float*)wuv, nw, rotab,
                              (float*)rows, pos, table, (float*)qa, part_o,
-                             part_ml, B, W, bs_log, g, eps, splits, stream);
+                             part_ml, B, W, bs_log, g, eps, splits, tile, stream);
   return run_decode<u16>((u16*)out, os, (const u16*)proj, ps,
                          (const u16*)wuk, (const u16*)wuv, nw, rotab,
                          (u16*)rows, pos, table, (u16*)qa, part_o, part_ml, B,
-                         W, bs_log, g, eps, splits, stream);
+                         W, bs_log, g, eps, splits, tile, stream);
 }
 
 void fei_latent_append(void* proj, long ps, void* rows, const float* nw,

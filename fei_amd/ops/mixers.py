@@ -19,8 +19,7 @@ _c = ctypes
 _vp, _i, _f, _l = _c.c_void_p, _c.c_int, _c.c_float, _c.c_long
 
 MAX_SPLITS = 64          # splits of a decode row's keys
-KEYS_PER_SPLIT = 64
-TARGET_BLOCKS = 512      # workgroups of a decode attention launch
+TARGET_BLOCKS = 256      # workgroups of a decode attention launch
 
 
 def declare(lib: ctypes.CDLL) -> None:
@@ -32,7 +31,8 @@ def declare(lib: ctypes.CDLL) -> None:
     lib.fei_gemv_f32.argtypes = [_vp] * 4 + [_i] * 3 + [_i, _f, _f, _i, _vp]
     lib.fei_gemm_m8_f32.argtypes = [_vp] * 4 + [_i] * 4 + [_f, _f, _vp]
     lib.fei_latent_decode.argtypes = (
-        [_vp, _l, _vp, _l] + [_vp] * 10 + [_i] * 8 + [_f, _i, _f, _i, _i, _vp])
+        [_vp, _l, _vp, _l] + [_vp] * 10 + [_i] * 8 +
+        [_f, _i, _f, _i, _i, _i, _vp])
     lib.fei_latent_decode.restype = _i
     lib.fei_latent_append.argtypes = (
         [_vp, _l] + [_vp] * 6 + [_i] * 8 + [_f, _i, _vp])
@@ -52,7 +52,8 @@ def _lib() -> ctypes.CDLL:
 
 
 def _stream() -> int:
-    return torch.cuda.current_stream().cuda_stream
+    from fei_amd import ops
+    return ops._stream()
 
 
 def _p(t: Optional[torch.Tensor]):
@@ -146,27 +147,28 @@ def mix_in(n1: torch.Tensor, n2: Optional[torch.Tensor], w_in: torch.Tensor,
 
 def _mm_f32(a: torch.Tensor, w: torch.Tensor,
             add: Optional[torch.Tensor]) -> torch.Tensor:
-    """a @ w^T (+ add) with a float32 result."""
+    """a @ w^T (+ add) with a float32 result; a 2-d ``add`` may be
+    overwritten with it."""
     if not a.is_cuda or a.dtype == torch.float32:
         y = torch.nn.functional.linear(a.float(), w.float())
         return y if add is None else add + y
     if add is None:
         return torch.mm(a, w.t(), out_dtype=torch.float32)
     if add.dim() == 1:
-        add = add.expand(a.shape[0], -1)
-    return torch.addmm(add, a, w.t(), out_dtype=torch.float32)
+        return torch.addmm(add.expand(a.shape[0], -1), a, w.t(),
+                           out_dtype=torch.float32)
+    return torch.addmm(add, a, w.t(), out_dtype=torch.float32, out=add)
 
 
 def residual_linear(x: torch.Tensor, a: torch.Tensor,
                     w: torch.Tensor) -> torch.Tensor:
-    """x + a @ w^T, float32."""
+    """x + a @ w^T, float32; x may be overwritten with it."""
     T, K = a.shape
     if a.is_cuda and _m8(T, K, a, w.shape[0]):
         _lib().fei_gemm_m8_f32(_p(x), _p(a), _p(w), None, T, w.shape[0], K, 1,
                                1.0, 0.0, _stream())
         return x
     if a.is_cuda and _gemv_rows(T, K, a):
-        # in place on x: the caller's residual is dead after this
         _lib().fei_gemv_f32(_p(x), _p(a), _p(w), None, T, w.shape[0], K, 1,
                             1.0, 0.0, 1, _stream())
         return x
@@ -265,8 +267,10 @@ def latent_attn_decode(proj, out, m, w, rot, batch, rows,
     if m.window is not None:
         n_max = min(n_max, m.window)
     groups = B * -(-m.heads // 16)
-    splits = max(1, min(MAX_SPLITS, -(-n_max // KEYS_PER_SPLIT),
+    splits = max(1, min(MAX_SPLITS, -(-n_max // 16),
                         -(-TARGET_BLOCKS // groups)))
+    per_split = -(-n_max // splits)
+    tile = 16 if per_split <= 16 else 32 if per_split <= 32 else 64
     qa = torch.empty(B, m.heads, m.row_width, dtype=proj.dtype, device=dev)
     part_o = torch.empty(B, m.heads, splits, m.kv_rank, dtype=torch.float32,
                          device=dev)
@@ -277,7 +281,7 @@ def latent_attn_decode(proj, out, m, w, rot, batch, rows,
         _p(w.norm), _p(rot), _p(rows), _p(batch.pos), _p(batch.table), _p(qa),
         _p(part_o), _p(part_ml), B, W, block_size.bit_length() - 1, m.heads,
         m.dim, m.rot_dim, m.vdim, m.kv_rank, m.scale, m.window or 0, w.eps,
-        splits, _f32(proj), _stream())
+        splits, tile, _f32(proj), _stream())
     if rc:
         raise ValueError(f"no decode tile for {m}")
 
