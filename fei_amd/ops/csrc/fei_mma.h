@@ -26,14 +26,24 @@ template <typename T> struct El;
 template <> struct El<u16> {
   typedef s16x8 frag;
   static __device__ __forceinline__ float ld(u16 v) { return bf2f(v); }
-  static __device__ __forceinline__ u16 st(float v) { return f2bf(v); }
+  // the hardware's conversion, round to nearest even
+  static __device__ __forceinline__ u16 st(float v) {
+    return __builtin_bit_cast(u16, (__bf16)v);
+  }
   static __device__ __forceinline__ float ex(float x) { return __expf(x); }
+  // exp(x) of an x that was scaled by ``base``
+  static constexpr float base = 1.44269504088896340736f;   // log2(e)
+  static __device__ __forceinline__ float exb(float x) {
+    return __builtin_amdgcn_exp2f(x);
+  }
 };
 template <> struct El<float> {
   typedef f32x8 frag;
   static __device__ __forceinline__ float ld(float v) { return v; }
   static __device__ __forceinline__ float st(float v) { return v; }
   static __device__ __forceinline__ float ex(float x) { return expf(x); }
+  static constexpr float base = 1.f;
+  static __device__ __forceinline__ float exb(float x) { return expf(x); }
 };
 
 // 8 consecutive elements at p (16-byte aligned in LDS and, where used, in
@@ -50,6 +60,27 @@ __device__ __forceinline__ void st8(float* p, f32x8 v) {
 }
 __device__ __forceinline__ float get8(s16x8 v, int j) { return bf2f((u16)v[j]); }
 __device__ __forceinline__ float get8(f32x8 v, int j) { return v[j]; }
+
+// Reductions over the 16 lanes of a DPP row (lanes 16i .. 16i+15), by
+// rotations: every lane gets the result, no LDS traffic.
+template <int N>
+__device__ __forceinline__ float row_ror(float v) {
+  return __builtin_bit_cast(
+      float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v),
+                                         0x120 + N, 0xf, 0xf, true));
+}
+__device__ __forceinline__ float row16_max(float v) {
+  v = fmaxf(v, row_ror<8>(v));
+  v = fmaxf(v, row_ror<4>(v));
+  v = fmaxf(v, row_ror<2>(v));
+  return fmaxf(v, row_ror<1>(v));
+}
+__device__ __forceinline__ float row16_sum(float v) {
+  v += row_ror<8>(v);
+  v += row_ror<4>(v);
+  v += row_ror<2>(v);
+  return v + row_ror<1>(v);
+}
 
 // Precise sigmoid and silu.
 __device__ __forceinline__ float sigmoid_f(float x) {

@@ -39,8 +39,8 @@ struct Gla {
   __device__ __host__ int a_off() const { return 2 * kq() + 2 * vo(); }
 };
 
-__device__ __forceinline__ float log_decay(float z, float tau) {
-  return (fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) / tau;
+__device__ __forceinline__ float log_decay(float z, float inv_tau) {
+  return (fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau;
 }
 
 // chunks [.][3]: portion, first row, rows. G [T][H dim].
@@ -59,6 +59,7 @@ k_gla_gate(float* __restrict__ G, const T* __restrict__ proj, long ps,
                            : 0.f;
   }
   __syncthreads();
+  const float inv_tau = 1.f / g.tau;
   const int cx = threadIdx.x & 63, sb = threadIdx.x >> 6;
   const int c = blockIdx.y * 64 + cx;
   float z[16];
@@ -74,7 +75,7 @@ k_gla_gate(float* __restrict__ G, const T* __restrict__ proj, long ps,
     float sum = 0.f;
 #pragma unroll
     for (int t = 0; t < 16; ++t) {
-      sum += log_decay(z[t], g.tau);
+      sum += log_decay(z[t], inv_tau);
       z[t] = sum;
     }
     tot[sb][cx] = sum;
@@ -90,22 +91,69 @@ k_gla_gate(float* __restrict__ G, const T* __restrict__ proj, long ps,
   }
 }
 
-// V^T tile [ne][CH + 8] of value columns e0 .. e0+ne-1, zero past the chunk
-// and past vdim. Four tokens per store, lanes along the columns.
+// A tile held transposed, [column][64 tokens] float32: the 16-byte blocks of
+// a column are permuted by the column, so that stores with lanes along the
+// columns' quads and reads of one block of 16 columns both spread over the
+// banks.
+__device__ __forceinline__ int tr_at(int col, int blk) {
+  return col * CH + ((blk ^ ((col >> 2) & 15) ^ ((col & 3) << 2)) << 2);
+}
+__device__ __forceinline__ f32x8 tr_ld8(const float* tile, int col, int t) {
+  const f32x4 a = *(const f32x4*)(tile + tr_at(col, t >> 2));
+  const f32x4 b = *(const f32x4*)(tile + tr_at(col, (t >> 2) + 1));
+  return f32x8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+}
+
+// 4 consecutive elements of a row; with vec their place is 8- or 16-byte
+// aligned. Elements from ``lim`` on are zero.
 template <typename T>
+__device__ __forceinline__ f32x4 ld4(const T* p, int lim, int vec) {
+  f32x4 v = {0.f, 0.f, 0.f, 0.f};
+  if (vec) {
+    if (lim > 0) {
+      T t[4];
+      __builtin_memcpy(t, __builtin_assume_aligned(p, 4 * sizeof(T)),
+                       sizeof(t));
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] = El<T>::ld(t[j]);
+    }
+  } else {
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (j < lim) v[j] = El<T>::ld(p[j]);
+  }
+  return v;
+}
+
+// Values of columns e0 .. e0+NE-1, transposed, zero past the chunk and past
+// vdim. A thread turns 4 tokens x 4 columns.
+template <typename T, int NE>
 __device__ __forceinline__ void stage_vt(float* vt, const T* __restrict__ proj,
                                          long ps, const Gla& g, int h, int row0,
-                                         int n, int e0, int ne) {
-  for (int i = threadIdx.x; i < ne * (CH / 4); i += 256) {
-    const int e = i % ne, t = i / ne * 4;
-    f32x4 v = {0.f, 0.f, 0.f, 0.f};
-    if (e0 + e < g.vdim)
+                                         int n, int e0, int vec) {
+  constexpr int Q = NE / 4;
+  constexpr int NU = (Q * 16 + 255) / 256;
+  f32x4 x[NU][4];
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (t + j < n)
-          v[j] = El<T>::ld(proj[(long)(row0 + t + j) * ps + g.v_off() +
-                                h * g.vdim + e0 + e]);
-    *(f32x4*)(vt + e * (CH + 8) + t) = v;
+  for (int u = 0; u < NU; ++u) {
+    const int i = threadIdx.x + u * 256;
+    const int e = i % Q * 4, t = i / Q * 4;
+    const int lim = i < Q * 16 ? g.vdim - e0 - e : 0;
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      x[u][j] = ld4<T>(proj + (long)(row0 + min(t + j, n - 1)) * ps +
+                           g.v_off() + h * g.vdim + e0 + e,
+                       t + j < n ? lim : 0, vec);
+  }
+#pragma unroll
+  for (int u = 0; u < NU; ++u) {
+    const int i = threadIdx.x + u * 256;
+    const int e = i % Q * 4, t = i / Q * 4;
+    if (i < Q * 16)
+#pragma unroll
+      for (int c = 0; c < 4; ++c)
+        *(f32x4*)(vt + tr_at(e + c, t >> 2)) =
+            f32x4{x[u][0][c], x[u][1][c], x[u][2][c], x[u][3][c]};
   }
 }
 
@@ -115,29 +163,39 @@ template <typename T, int DT>              // DT = ceil(dim / 16), rounded up
 __global__ void __launch_bounds__(256)
 k_gla_state(float* __restrict__ U, const float* __restrict__ G,
             const T* __restrict__ proj, long ps,
-            const int* __restrict__ chunks, Gla g) {
+            const int* __restrict__ chunks, Gla g, int vec) {
   extern __shared__ __align__(16) char smem[];
-  float* kt = (float*)smem;                // [DT * 16][CH + 8]
-  float* vt = kt + DT * 16 * (CH + 8);     // [64][CH + 8]
+  float* kt = (float*)smem;                // [DT * 16][CH], see tr_at
+  float* vt = kt + DT * 16 * CH;           // [64][CH]
   const int row0 = chunks[blockIdx.x * 3 + 1], n = chunks[blockIdx.x * 3 + 2];
   const int h = blockIdx.y, e0 = blockIdx.z * 64;
   const float* gend = G + (long)(row0 + n - 1) * g.kq() + h * g.dim;
-  for (int i = threadIdx.x; i < DT * 16 * (CH / 4); i += 256) {
-    const int d = i % (DT * 16), t = i / (DT * 16) * 4;
-    f32x4 v = {0.f, 0.f, 0.f, 0.f};
-    if (d < g.dim) {
-      const float ge = gend[d];
+  constexpr int Q = DT * 4;                // quads of channels
+  constexpr int NU = (Q * 16 + 255) / 256;
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (t + j < n) {
-          const long row = row0 + t + j;
-          v[j] = El<T>::ld(proj[row * ps + g.k_off() + h * g.dim + d]) *
-                 expf(ge - G[row * g.kq() + h * g.dim + d]);
-        }
+  for (int u = 0; u < NU; ++u) {
+    const int i = threadIdx.x + u * 256;
+    const int d = i % Q * 4, t = i / Q * 4;
+    const int lim = i < Q * 16 ? g.dim - d : 0;
+    const f32x4 ge = ld4<float>(gend + d, lim, vec);
+    f32x4 k[4], gg[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const long row = row0 + min(t + j, n - 1);
+      k[j] = ld4<T>(proj + row * ps + g.k_off() + h * g.dim + d,
+                    t + j < n ? lim : 0, vec);
+      gg[j] = ld4<float>(G + row * g.kq() + h * g.dim + d, lim, vec);
     }
-    *(f32x4*)(kt + d * (CH + 8) + t) = v;
+    if (i < Q * 16)
+#pragma unroll
+      for (int c = 0; c < 4; ++c) {
+        f32x4 v;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[j] = k[j][c] * El<T>::ex(ge[c] - gg[j][c]);
+        *(f32x4*)(kt + tr_at(d + c, t >> 2)) = v;
+      }
   }
-  stage_vt<T>(vt, proj, ps, g, h, row0, n, e0, 64);
+  stage_vt<T, 64>(vt, proj, ps, g, h, row0, n, e0, vec);
   __syncthreads();
   const int w = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int l15 = lane & 15, lg = lane >> 4;
@@ -145,15 +203,14 @@ k_gla_state(float* __restrict__ U, const float* __restrict__ G,
   f32x8 a[2];
 #pragma unroll
   for (int k = 0; k < 2; ++k)
-    a[k] = ld8(vt + (w * 16 + l15) * (CH + 8) + k * 32 + 8 * lg);
+    a[k] = tr_ld8(vt, w * 16 + l15, k * 32 + 8 * lg);
   float* u = U + ((long)blockIdx.x * g.heads + h) * g.vdim * g.dim;
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt) {
     f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int k = 0; k < 2; ++k)
-      acc = mma(a[k], ld8(kt + (dt * 16 + l15) * (CH + 8) + k * 32 + 8 * lg),
-                acc);
+      acc = mma(a[k], tr_ld8(kt, dt * 16 + l15, k * 32 + 8 * lg), acc);
     const int d = dt * 16 + l15;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
@@ -205,7 +262,7 @@ template <typename T>
 __global__ void __launch_bounds__(256)
 k_gla_scores(float* __restrict__ A, const float* __restrict__ G,
              const T* __restrict__ proj, long ps,
-             const int* __restrict__ chunks, Gla g) {
+             const int* __restrict__ chunks, Gla g, int vec) {
   constexpr int DS = 64 + 4;
   __shared__ __align__(16) float qs[CH * DS], ks[CH * DS], gs[CH * DS];
   const int row0 = chunks[blockIdx.x * 3 + 1], n = chunks[blockIdx.x * 3 + 2];
@@ -220,21 +277,27 @@ k_gla_scores(float* __restrict__ A, const float* __restrict__ G,
 
   for (int d0 = 0; d0 < g.dim; d0 += 64) {
     __syncthreads();
-    for (int i = threadIdx.x; i < CH * 64; i += 256) {
-      const int t = i >> 6, d = i & 63;
-      float q = 0.f, k = 0.f, gg = 0.f;
-      if (d0 + d < g.dim) {
+    {
+      f32x4 q[4], k[4], gg[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int i = threadIdx.x + u * 256;
+        const int t = i >> 4, d = d0 + (i & 15) * 4;
         // past the chunk: G of the last token, so that no exponent is positive
-        gg = G[(long)(row0 + min(t, n - 1)) * g.kq() + h * g.dim + d0 + d];
-        if (t < n) {
-          const T* pr = proj + (long)(row0 + t) * ps + h * g.dim + d0 + d;
-          q = El<T>::ld(pr[0]) * scale;
-          k = El<T>::ld(pr[g.k_off()]);
-        }
+        const long row = row0 + min(t, n - 1);
+        const int lim = g.dim - d, on = t < n ? lim : 0;
+        q[u] = ld4<T>(proj + row * ps + h * g.dim + d, on, vec);
+        k[u] = ld4<T>(proj + row * ps + g.k_off() + h * g.dim + d, on, vec);
+        gg[u] = ld4<float>(G + row * g.kq() + h * g.dim + d, lim, vec);
       }
-      qs[t * DS + d] = q;
-      ks[t * DS + d] = k;
-      gs[t * DS + d] = gg;
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int i = threadIdx.x + u * 256;
+        const int at = (i >> 4) * DS + (i & 15) * 4;
+        *(f32x4*)(qs + at) = q[u] * scale;
+        *(f32x4*)(ks + at) = k[u];
+        *(f32x4*)(gs + at) = gg[u];
+      }
     }
     __syncthreads();
     if (w > 0) {
@@ -245,14 +308,14 @@ k_gla_scores(float* __restrict__ A, const float* __restrict__ G,
         f32x8 a = ld8(qs + (w * 16 + l15) * DS + c);
         const f32x8 ga = ld8(gs + (w * 16 + l15) * DS + c);
 #pragma unroll
-        for (int j = 0; j < 8; ++j) a[j] *= expf(ga[j] - ref[j]);
+        for (int j = 0; j < 8; ++j) a[j] *= El<T>::ex(ga[j] - ref[j]);
 #pragma unroll
         for (int jb = 0; jb < 3; ++jb)
           if (jb < w) {
             f32x8 b = ld8(ks + (jb * 16 + l15) * DS + c);
             const f32x8 gb = ld8(gs + (jb * 16 + l15) * DS + c);
 #pragma unroll
-            for (int j = 0; j < 8; ++j) b[j] *= expf(ref[j] - gb[j]);
+            for (int j = 0; j < 8; ++j) b[j] *= El<T>::ex(ref[j] - gb[j]);
             off[jb] = mma(a, b, off[jb]);
           }
       }
@@ -268,7 +331,8 @@ k_gla_scores(float* __restrict__ A, const float* __restrict__ G,
         const f32x4 g4 = *(const f32x4*)(gs + s * DS + d);
 #pragma unroll
         for (int j = 0; j < 4; ++j)        // s > t is dropped below
-          diag[r] = fmaf(q4[j] * k4[j], expf(fminf(gt[j] - g4[j], 0.f)), diag[r]);
+          diag[r] = fmaf(q4[j] * k4[j], El<T>::ex(fminf(gt[j] - g4[j], 0.f)),
+                         diag[r]);
       }
     }
   }
@@ -293,10 +357,10 @@ __global__ void __launch_bounds__(256)
 k_gla_out(T* __restrict__ out, long os, const float* __restrict__ S,
           const float* __restrict__ A, const float* __restrict__ G,
           const T* __restrict__ proj, long ps, const float* __restrict__ nw,
-          const int* __restrict__ chunks, Gla g, float eps) {
+          const int* __restrict__ chunks, Gla g, float eps, int vec) {
   constexpr int DS = DK * 32 + 4;
   __shared__ __align__(16) float st[32 * DS];
-  __shared__ __align__(16) float vt[32 * (CH + 8)];
+  __shared__ __align__(16) float vt[32 * CH];
   const int row0 = chunks[blockIdx.x * 3 + 1], n = chunks[blockIdx.x * 3 + 2];
   const int h = blockIdx.y;
   const int w = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -307,16 +371,19 @@ k_gla_out(T* __restrict__ out, long os, const float* __restrict__ S,
   f32x8 aq[DK], aa[2];
   const int t = w * 16 + l15;
 #pragma unroll
-  for (int k = 0; k < DK; ++k)
+  for (int k = 0; k < DK; ++k) {
+    const long row = row0 + min(t, n - 1);
+    const int d = k * 32 + 8 * lg;
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      const int d = k * 32 + 8 * lg + j;
-      float v = 0.f;
-      if (t < n && d < g.dim)
-        v = El<T>::ld(proj[(long)(row0 + t) * ps + h * g.dim + d]) * scale *
-            expf(G[(long)(row0 + t) * g.kq() + h * g.dim + d]);
-      aq[k][j] = v;
+    for (int b = 0; b < 2; ++b) {
+      const int lim = t < n ? g.dim - d - 4 * b : 0;
+      const f32x4 q = ld4<T>(proj + row * ps + h * g.dim + d + 4 * b, lim, vec);
+      const f32x4 gg = ld4<float>(G + row * g.kq() + h * g.dim + d + 4 * b, lim,
+                                  vec);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) aq[k][4 * b + j] = q[j] * scale * El<T>::ex(gg[j]);
     }
+  }
 #pragma unroll
   for (int k = 0; k < 2; ++k)
     aa[k] = ld8(A + (((long)blockIdx.x * g.heads + h) * CH + t) * CH + k * 32 +
@@ -328,12 +395,20 @@ k_gla_out(T* __restrict__ out, long os, const float* __restrict__ S,
     const int e0 = v * 32;
     if (e0 < g.vdim) {                     // uniform
       __syncthreads();
-      for (int i = threadIdx.x; i < 32 * DK * 32; i += 256) {
-        const int e = i / (DK * 32), d = i - e * (DK * 32);
-        st[e * DS + d] = (e0 + e < g.vdim && d < g.dim)
-                             ? s0[(long)(e0 + e) * g.dim + d] : 0.f;
+      f32x4 x[DK];
+#pragma unroll
+      for (int u = 0; u < DK; ++u) {
+        const int i = threadIdx.x + u * 256;
+        const int e = i / (DK * 8), d = i % (DK * 8) * 4;
+        x[u] = ld4<float>(s0 + (long)(e0 + e) * g.dim + d,
+                          e0 + e < g.vdim ? g.dim - d : 0, vec);
       }
-      stage_vt<T>(vt, proj, ps, g, h, row0, n, e0, 32);
+#pragma unroll
+      for (int u = 0; u < DK; ++u) {
+        const int i = threadIdx.x + u * 256;
+        *(f32x4*)(st + i / (DK * 8) * DS + i % (DK * 8) * 4) = x[u];
+      }
+      stage_vt<T, 32>(vt, proj, ps, g, h, row0, n, e0, vec);
       __syncthreads();
 #pragma unroll
       for (int c = 0; c < 2; ++c) {
@@ -343,8 +418,7 @@ k_gla_out(T* __restrict__ out, long os, const float* __restrict__ S,
           acc = mma(aq[k], ld8(st + (c * 16 + l15) * DS + k * 32 + 8 * lg), acc);
 #pragma unroll
         for (int k = 0; k < 2; ++k)
-          acc = mma(aa[k], ld8(vt + (c * 16 + l15) * (CH + 8) + k * 32 + 8 * lg),
-                    acc);
+          acc = mma(aa[k], tr_ld8(vt, c * 16 + l15, k * 32 + 8 * lg), acc);
         o[v * 2 + c] = acc;
       }
     } else {
@@ -356,8 +430,7 @@ k_gla_out(T* __restrict__ out, long os, const float* __restrict__ S,
     float ss = 0.f;                        // columns past vdim are zero
 #pragma unroll
     for (int c = 0; c < NV * 2; ++c) ss = fmaf(o[c][r], o[c][r], ss);
-#pragma unroll
-    for (int off = 1; off < 16; off <<= 1) ss += __shfl_xor(ss, off);
+    ss = row16_sum(ss);
     const int tr = w * 16 + 4 * lg + r;
     if (tr >= n) continue;
     const float inv = 1.f / sqrtf(ss / (float)g.vdim + eps);
@@ -394,7 +467,7 @@ k_gla_decode(float* __restrict__ o, float* __restrict__ states,
     const int c = h * g.dim + tid;
     float z = bias[c];
     for (int r = 0; r < g.rank; ++r) z = fmaf(a2[(long)c * g.rank + r], a1[r], z);
-    al[tid] = expf(log_decay(z, g.tau));
+    al[tid] = expf(log_decay(z, 1.f / g.tau));
     q[tid] = El<T>::ld(pr[c]) / sqrtf((float)g.dim);
     k[tid] = El<T>::ld(pr[g.k_off() + c]);
   }
@@ -470,8 +543,9 @@ void run_gla_decode(T* out, long os, float* o, float* states, const T* proj,
 
 template <typename T, int DT>
 void launch_state(float* U, const float* G, const T* proj, long ps,
-                  const int* chunks, int n, Gla g, hipStream_t stream) {
-  const size_t lds = 4 * (DT * 16 + 64) * (CH + 8);
+                  const int* chunks, int n, Gla g, int vec,
+                  hipStream_t stream) {
+  const size_t lds = 4 * (DT * 16 + 64) * CH;
   static bool set = false;
   if (!set) {
     (void)hipFuncSetAttribute((const void*)k_gla_state<T, DT>,
@@ -481,7 +555,7 @@ void launch_state(float* U, const float* G, const T* proj, long ps,
   }
   hipLaunchKernelGGL((k_gla_state<T, DT>),
                      dim3(n, g.heads, (g.vdim + 63) / 64), dim3(256), lds,
-                     stream, U, G, proj, ps, chunks, g);
+                     stream, U, G, proj, ps, chunks, g, vec);
 }
 
 template <typename T>
@@ -492,20 +566,23 @@ void run_gla_prefill(T* out, long os, const T* proj, long ps, const float* a2,
                      float eps, hipStream_t stream) {
   hipLaunchKernelGGL(k_gla_gate<T>, dim3(n, (g.kq() + 63) / 64), dim3(256),
                      4 * CH * g.rank, stream, G, proj, ps, a2, bias, chunks, g);
+  // quads of q, k, v, G and S lie on 8- and 16-byte borders
+  const int vec = g.dim % 4 == 0 && g.vdim % 4 == 0 && ps % 4 == 0 &&
+                  (size_t)proj % 16 == 0;
   const int dt = (g.dim + 15) / 16;
-  if (dt <= 2) launch_state<T, 2>(U, G, proj, ps, chunks, n, g, stream);
-  else if (dt <= 4) launch_state<T, 4>(U, G, proj, ps, chunks, n, g, stream);
-  else if (dt <= 8) launch_state<T, 8>(U, G, proj, ps, chunks, n, g, stream);
-  else launch_state<T, 16>(U, G, proj, ps, chunks, n, g, stream);
+  if (dt <= 2) launch_state<T, 2>(U, G, proj, ps, chunks, n, g, vec, stream);
+  else if (dt <= 4) launch_state<T, 4>(U, G, proj, ps, chunks, n, g, vec, stream);
+  else if (dt <= 8) launch_state<T, 8>(U, G, proj, ps, chunks, n, g, vec, stream);
+  else launch_state<T, 16>(U, G, proj, ps, chunks, n, g, vec, stream);
   const long size = (long)g.heads * g.vdim * g.dim;
   hipLaunchKernelGGL(k_gla_scan, dim3((size + 255) / 256, P), dim3(256), 0,
                      stream, U, G, states, chunks, spans, slots, g);
   hipLaunchKernelGGL(k_gla_scores<T>, dim3(n, g.heads), dim3(256), 0, stream,
-                     A, G, proj, ps, chunks, g);
+                     A, G, proj, ps, chunks, g, vec);
   const dim3 go(n, g.heads);
 #define OUT(DK, NV)                                                         \
   hipLaunchKernelGGL((k_gla_out<T, DK, NV>), go, dim3(256), 0, stream, out, \
-                     os, U, A, G, proj, ps, nw, chunks, g, eps)
+                     os, U, A, G, proj, ps, nw, chunks, g, eps, vec)
 #define BY_NV(DK)                           \
   do {                                      \
     if (g.vdim <= 64) OUT(DK, 2);           \

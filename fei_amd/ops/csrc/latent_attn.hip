@@ -311,8 +311,7 @@ k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
         }
         mx = fmaxf(mx, sv[i]);
       }
-#pragma unroll
-      for (int off = 1; off < 16; off <<= 1) mx = fmaxf(mx, __shfl_xor(mx, off));
+      mx = row16_max(mx);
       const float a = El<T>::ex(m - mx);   // a tile has a visible key: mx is finite
       float sum = 0.f;
 #pragma unroll
@@ -326,9 +325,7 @@ k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
             ph[(pi * 16 + row) * KPs + c] = part_of<T>(e, pi);
         }
       }
-#pragma unroll
-      for (int off = 1; off < 16; off <<= 1) sum += __shfl_xor(sum, off);
-      l = l * a + sum;
+      l = l * a + row16_sum(sum);
       m = mx;
       if (l15 == 0) al[row] = a;
     }
@@ -487,230 +484,228 @@ __device__ __forceinline__ int vt_at(int col, int key) {
 }
 
 // Flash attention of prompt portions over expanded keys and values.
-// grid (heads, query tiles), 4 waves; a wave owns MR tiles of 16 query rows,
-// the block 64*MR of them, in tiles of 64 keys held in LDS: keys row-major,
+// grid (heads, query tiles), NW waves; a wave owns 16 query rows, and the
+// block walks the keys they see in tiles of 64 held in LDS: keys row-major,
 // values transposed. tiles [.][2]: portion, first row in it (a tile of the
-// plan is 128 rows; with MR = 1 two blocks share it, blockIdx.z).
+// plan is 128 rows; with 4 waves two blocks share it, blockIdx.z).
 // KS = ceil((dim + rot) / 32), DC = ceil(vdim / 16), rounded up to what is
-// instantiated; zero padding in LDS makes the padded products vanish.
-template <typename T, int KS, int DC, int MR>
-__global__ void __launch_bounds__(256, 2)
+// instantiated; queries are zero beyond dim + rot, columns beyond vdim are
+// not stored.
+template <typename T, int KS, int DC, int NW>
+__global__ void __launch_bounds__(NW * 64, 2)
 k_window_prefill(T* __restrict__ out, long os, const T* __restrict__ proj,
                  long ps, const T* __restrict__ kv, const T* __restrict__ krot,
                  const int* __restrict__ spans, const int* __restrict__ tiles,
                  int gate_off, Geo g, int vec) {
   typedef typename El<T>::frag frag;
   constexpr int NP = Parts<T>::n;
+  constexpr int NT = NW * 64;
   constexpr int DS = KS * 32 + 8;          // odd count of 16-byte slots
   constexpr int PS = 64 + 8;
   extern __shared__ __align__(16) char smem[];
   T* kt = (T*)smem;                        // [64][DS]
   T* vt = kt + 64 * DS;                    // [DC * 16][64], see vt_at
-  T* pl = vt + DC * 16 * 64;               // [4 waves][NP][16][PS]
+  T* pl = vt + DC * 16 * 64;               // [NW][NP][16][PS]
 
   // heads run fastest, so that with 8 | heads a head stays on one XCD and
   // neighbouring tiles find their common keys in its L2
   const int h = blockIdx.x;
   const int* sp = spans + tiles[blockIdx.y * 2] * 5;
   const int row0 = sp[0], cnt = sp[1], pos0 = sp[2], key0 = sp[3], at0 = sp[4];
-  const int q0 = tiles[blockIdx.y * 2 + 1] + (MR == 1 ? blockIdx.z * 64 : 0);
+  const int q0 = tiles[blockIdx.y * 2 + 1] + blockIdx.z * NW * 16;
   if (q0 >= cnt) return;
-  const int qn = min(64 * MR, cnt - q0);
+  const int qn = min(16 * NW, cnt - q0);
   const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63;
   const int l15 = lane & 15, lg = lane >> 4;
   const int D = g.dim + g.rot;
   const long kvs = (long)g.heads * (g.dim + g.vdim);
+  const T* kh = kv + (long)h * g.dim;
+  const T* vh = kv + (long)g.heads * g.dim + (long)h * g.vdim;
 
-  // queries: row i*64 + w*16 + l15 of the tile
-  frag aq[MR][KS];
-#pragma unroll
-  for (int i = 0; i < MR; ++i) {
-    const int r = min(i * 64 + w * 16 + l15, qn - 1);
+  frag aq[KS];
+  {
+    const int r = min(w * 16 + l15, qn - 1);
     const T* q = proj + (long)(row0 + q0 + r) * ps + (long)h * D;
 #pragma unroll
     for (int k = 0; k < KS; ++k) {
       const int c = k * 32 + 8 * lg;
-      frag f;
-      if (vec && c + 8 <= D) {
-        f = ld8(q + c);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) aq[k][j] = 0;
+      if (vec) {
+        if (c < D) aq[k] = ld8(q + c);
       } else {
 #pragma unroll
         for (int j = 0; j < 8; ++j)
-          f[j] = c + j < D ? q[c + j] : El<T>::st(0.f);
+          if (c + j < D) aq[k][j] = q[c + j];
       }
-      aq[i][k] = f;
     }
   }
-  float m[MR][4], l[MR][4];
-  f32x4 o[MR][DC];
+  float m[4], l[4];
+  f32x4 o[DC];
 #pragma unroll
-  for (int i = 0; i < MR; ++i) {
+  for (int r = 0; r < 4; ++r) { m[r] = NEG_INF; l[r] = 0.f; }
 #pragma unroll
-    for (int r = 0; r < 4; ++r) { m[i][r] = NEG_INF; l[i][r] = 0.f; }
-#pragma unroll
-    for (int d = 0; d < DC; ++d) o[i][d] = f32x4{0.f, 0.f, 0.f, 0.f};
-  }
+  for (int d = 0; d < DC; ++d) o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
 
   // positions of this tile's queries and of the keys any of them sees
   const int qa = pos0 + q0, qb = qa + qn - 1;
   const int klo = max(first_key(qa, g.window), key0) & ~63;
+  // this wave's own range: tiles outside it are staged for the others only
+  const int wa = qa + w * 16, wb = min(wa + 15, qb);
+  const int wlo = first_key(wa, g.window);
   T* pw = pl + w * NP * 16 * PS;
+  const float scale = g.scale * El<T>::base;
 
   for (int t0 = klo; t0 <= qb; t0 += 64) {
     __syncthreads();
-    // keys [64][KS*32]
     if (vec) {
-      constexpr int NV = KS * 4;
-      for (int i = tid; i < 64 * NV; i += 256) {
+      // all loads before the first store. Keys outside the range and columns
+      // past the head's sizes read some valid place: the queries are zero
+      // there, the scores masked, the output columns dropped.
+      constexpr int NV = KS * 4, NC = DC * 2;
+      constexpr int UK = (64 * NV + NT - 1) / NT, UV = (32 * NC + NT - 1) / NT;
+      frag kf[UK], va[UV], vb[UV];
+#pragma unroll
+      for (int u = 0; u < UK; ++u) {
+        const int i = tid + u * NT;
         const int r = i / NV, c = (i - r * NV) * 8;
-        const int key = t0 + r;
-        frag v;
-#pragma unroll
-        for (int j = 0; j < 8; ++j) v[j] = 0;
-        if (key >= key0 && key <= qb && c < D) {
-          const long n = at0 + key - key0;
-          v = c < g.dim ? ld8(kv + n * kvs + (long)h * g.dim + c)
-                        : ld8(krot + n * g.rot + c - g.dim);
-        }
-        st8(kt + r * DS + c, v);
+        const int n = at0 + min(max(t0 + r, key0), qb) - key0;
+        const T* src = c >= g.dim && c < D
+                           ? krot + (long)n * g.rot + c - g.dim
+                           : kh + (long)n * kvs + (c < g.dim ? c : 0);
+        kf[u] = ld8(src);
       }
-      // values, two keys at a time so that a transposed store is a pair
-      constexpr int NW = DC * 2;
-      for (int i = tid; i < 32 * NW; i += 256) {
-        const int r = i / NW * 2, c = i % NW * 8;
-        frag a, bb;
 #pragma unroll
-        for (int j = 0; j < 8; ++j) { a[j] = 0; bb[j] = 0; }
-        if (c < g.vdim) {
-          const T* v = kv + (long)(at0 + t0 + r - key0) * kvs +
-                       (long)g.heads * g.dim + (long)h * g.vdim + c;
-          if (t0 + r >= key0 && t0 + r <= qb) a = ld8(v);
-          if (t0 + r + 1 >= key0 && t0 + r + 1 <= qb) bb = ld8(v + kvs);
-        }
+      for (int u = 0; u < UV; ++u) {
+        const int i = tid + u * NT;
+        const int r = i / NC * 2, c = min(i % NC * 8, g.vdim - 8);
+        const int ka = min(max(t0 + r, key0), qb) - key0;
+        const int kb = min(max(t0 + r + 1, key0), qb) - key0;
+        va[u] = ld8(vh + (long)(at0 + ka) * kvs + c);
+        vb[u] = ld8(vh + (long)(at0 + kb) * kvs + c);
+      }
 #pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          T two[2] = {(T)a[j], (T)bb[j]};
-          __builtin_memcpy(vt + vt_at(c + j, r), two, sizeof(two));
-        }
+      for (int u = 0; u < UK; ++u) {
+        const int i = tid + u * NT;
+        const int r = i / NV, c = (i - r * NV) * 8;
+        if (64 * NV % NT == 0 || i < 64 * NV) st8(kt + r * DS + c, kf[u]);
+      }
+#pragma unroll
+      for (int u = 0; u < UV; ++u) {
+        const int i = tid + u * NT;
+        const int r = i / NC * 2, c = i % NC * 8;
+        if (32 * NC % NT == 0 || i < 32 * NC)
+#pragma unroll
+          for (int j = 0; j < 8; ++j) {
+            T two[2] = {(T)va[u][j], (T)vb[u][j]};
+            __builtin_memcpy(vt + vt_at(c + j, r), two, sizeof(two));
+          }
       }
     } else {
-      for (int i = tid; i < 64 * KS * 32; i += 256) {
+      for (int i = tid; i < 64 * KS * 32; i += NT) {
         const int r = i / (KS * 32), c = i - r * (KS * 32);
         const int key = t0 + r;
         T v = El<T>::st(0.f);
         if (key >= key0 && key <= qb && c < D) {
           const long n = at0 + key - key0;
-          v = c < g.dim ? kv[n * kvs + (long)h * g.dim + c]
-                        : krot[n * g.rot + c - g.dim];
+          v = c < g.dim ? kh[n * kvs + c] : krot[n * g.rot + c - g.dim];
         }
         kt[r * DS + c] = v;
       }
-      for (int i = tid; i < 64 * DC * 16; i += 256) {
+      for (int i = tid; i < 64 * DC * 16; i += NT) {
         const int r = i / (DC * 16), c = i - r * (DC * 16);
         const int key = t0 + r;
         T v = El<T>::st(0.f);
         if (key >= key0 && key <= qb && c < g.vdim)
-          v = kv[(long)(at0 + key - key0) * kvs + (long)g.heads * g.dim +
-                 (long)h * g.vdim + c];
+          v = vh[(long)(at0 + key - key0) * kvs + c];
         vt[vt_at(c, r)] = v;
       }
     }
     __syncthreads();
+    if (t0 > wb || t0 + 63 < wlo) continue;
 
-    f32x4 s[MR][4];
+    f32x4 s[4];
 #pragma unroll
     for (int c = 0; c < 4; ++c) {
+      s[c] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int i = 0; i < MR; ++i) s[i][c] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int k = 0; k < KS; ++k) {
-        const frag bk = ld8(kt + (c * 16 + l15) * DS + k * 32 + 8 * lg);
-#pragma unroll
-        for (int i = 0; i < MR; ++i) s[i][c] = mma(aq[i][k], bk, s[i][c]);
-      }
+      for (int k = 0; k < KS; ++k)
+        s[c] = mma(aq[k], ld8(kt + (c * 16 + l15) * DS + k * 32 + 8 * lg), s[c]);
     }
-    // no mask where every query of the tile sees every key of the tile
-    const bool edge = t0 + 63 > qa || t0 < key0 ||
-                      (g.window > 0 && qb - t0 >= g.window);
+    // no mask where every query of the wave sees every key of the tile
+    const bool edge = t0 + 63 > wa || t0 < key0 ||
+                      (g.window > 0 && wb - t0 >= g.window);
+    float al[4];
 #pragma unroll
-    for (int i = 0; i < MR; ++i) {
-      float al[4];
+    for (int r = 0; r < 4; ++r) {
+      const int qp = wa + 4 * lg + r;
+      float mx = m[r];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int qp = qa + i * 64 + w * 16 + 4 * lg + r;
-        float mx = m[i][r];
-#pragma unroll
-        for (int c = 0; c < 4; ++c) {
-          float v = s[i][c][r] * g.scale;
-          if (edge) {
-            const int key = t0 + c * 16 + l15;
-            if (key > qp || key < key0 ||
-                (g.window > 0 && qp - key >= g.window))
-              v = NEG_INF;
-          }
-          s[i][c][r] = v;
-          mx = fmaxf(mx, v);
+      for (int c = 0; c < 4; ++c) {
+        float v = s[c][r] * scale;
+        if (edge) {
+          const int key = t0 + c * 16 + l15;
+          if (key > qp || key < key0 || (g.window > 0 && qp - key >= g.window))
+            v = NEG_INF;
         }
-#pragma unroll
-        for (int off = 1; off < 16; off <<= 1)
-          mx = fmaxf(mx, __shfl_xor(mx, off));
-        const bool any = mx > NEG_INF;     // no key so far: keep zeros
-        al[r] = any ? El<T>::ex(m[i][r] - mx) : 1.f;
-        m[i][r] = mx;
-        float sum = 0.f;
-#pragma unroll
-        for (int c = 0; c < 4; ++c) {
-          const float e = any ? El<T>::ex(s[i][c][r] - mx) : 0.f;
-          sum += e;
-#pragma unroll
-          for (int pi = 0; pi < NP; ++pi)
-            pw[(pi * 16 + 4 * lg + r) * PS + c * 16 + l15] = part_of<T>(e, pi);
-        }
-#pragma unroll
-        for (int off = 1; off < 16; off <<= 1) sum += __shfl_xor(sum, off);
-        l[i][r] = l[i][r] * al[r] + sum;
+        s[c][r] = v;
+        mx = fmaxf(mx, v);
       }
-      // pw belongs to this wave alone: its LDS operations stay in order
-      __builtin_amdgcn_wave_barrier();
-      frag ap[NP][2];
+      mx = row16_max(mx);
+      const bool any = mx > NEG_INF;       // no key so far: keep zeros
+      al[r] = any ? El<T>::exb(m[r] - mx) : 1.f;
+      m[r] = mx;
+      float sum = 0.f;                     // of this lane's columns
 #pragma unroll
-      for (int pi = 0; pi < NP; ++pi)
+      for (int c = 0; c < 4; ++c) {
+        const float e = any ? El<T>::exb(s[c][r] - mx) : 0.f;
+        sum += e;
 #pragma unroll
-        for (int k = 0; k < 2; ++k)
-          ap[pi][k] = ld8(pw + (pi * 16 + l15) * PS + k * 32 + 8 * lg);
-      __builtin_amdgcn_wave_barrier();
+        for (int pi = 0; pi < NP; ++pi)
+          pw[(pi * 16 + 4 * lg + r) * PS + c * 16 + l15] = part_of<T>(e, pi);
+      }
+      l[r] = fmaf(l[r], al[r], sum);
+    }
+    // pw belongs to this wave alone: its LDS operations stay in order
+    __builtin_amdgcn_wave_barrier();
+    frag ap[NP][2];
 #pragma unroll
-      for (int d = 0; d < DC; ++d) {
+    for (int pi = 0; pi < NP; ++pi)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) o[i][d][r] *= al[r];
+      for (int k = 0; k < 2; ++k)
+        ap[pi][k] = ld8(pw + (pi * 16 + l15) * PS + k * 32 + 8 * lg);
+    __builtin_amdgcn_wave_barrier();
 #pragma unroll
-        for (int k = 0; k < 2; ++k) {
-          const frag bv = ld8(vt + vt_at(d * 16 + l15, k * 32 + 8 * lg));
+    for (int d = 0; d < DC; ++d) {
 #pragma unroll
-          for (int pi = 0; pi < NP; ++pi)
-            o[i][d] = mma(ap[pi][k], bv, o[i][d]);
-        }
+      for (int r = 0; r < 4; ++r) o[d][r] *= al[r];
+#pragma unroll
+      for (int k = 0; k < 2; ++k) {
+        const frag bv = ld8(vt + vt_at(d * 16 + l15, k * 32 + 8 * lg));
+#pragma unroll
+        for (int pi = 0; pi < NP; ++pi) o[d] = mma(ap[pi][k], bv, o[d]);
       }
     }
   }
 
+  float lsum[4];
 #pragma unroll
-  for (int i = 0; i < MR; ++i)
+  for (int r = 0; r < 4; ++r) lsum[r] = row16_sum(l[r]);
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int q = i * 64 + w * 16 + 4 * lg + r;
-      if (q >= qn) continue;
-      const float inv = 1.f / l[i][r];     // a query always sees itself
-      const T* gate = proj + (long)(row0 + q0 + q) * ps + gate_off +
-                      (long)h * g.vdim;
-      T* dst = out + (long)(row0 + q0 + q) * os + (long)h * g.vdim;
+  for (int r = 0; r < 4; ++r) {
+    const int q = w * 16 + 4 * lg + r;
+    if (q >= qn) continue;
+    const float inv = 1.f / lsum[r];       // a query always sees itself
+    const T* gate = proj + (long)(row0 + q0 + q) * ps + gate_off +
+                    (long)h * g.vdim;
+    T* dst = out + (long)(row0 + q0 + q) * os + (long)h * g.vdim;
 #pragma unroll
-      for (int d = 0; d < DC; ++d) {
-        const int c = d * 16 + l15;
-        if (c < g.vdim)
-          dst[c] = El<T>::st(o[i][d][r] * inv * sigmoid_f(El<T>::ld(gate[c])));
-      }
+    for (int d = 0; d < DC; ++d) {
+      const int c = d * 16 + l15;
+      if (c < g.vdim)
+        dst[c] = El<T>::st(o[d][r] * inv * sigmoid_f(El<T>::ld(gate[c])));
     }
+  }
 }
 
 template <typename T>
@@ -776,19 +771,19 @@ template <typename T, int KS, int DC>
 void launch_window(T* out, long os, const T* proj, long ps, const T* kv,
                    const T* krot, const int* spans, const int* tiles,
                    int n_tiles, Geo g, int vec, hipStream_t stream) {
-  constexpr int MR = sizeof(T) == 2 && KS * 4 + DC * 4 <= 64 ? 2 : 1;
+  constexpr int NW = sizeof(T) == 2 ? 8 : 4;
   const size_t lds = sizeof(T) * (64 * (KS * 32 + 8) + DC * 16 * 64 +
-                                  4 * Parts<T>::n * 16 * 72);
+                                  NW * Parts<T>::n * 16 * 72);
   static bool set = false;
   if (!set) {
-    (void)hipFuncSetAttribute((const void*)k_window_prefill<T, KS, DC, MR>,
+    (void)hipFuncSetAttribute((const void*)k_window_prefill<T, KS, DC, NW>,
                               hipFuncAttributeMaxDynamicSharedMemorySize,
                               160 * 1024);
     set = true;
   }
-  const dim3 grid(g.heads, n_tiles, MR == 1 ? 2 : 1);
+  const dim3 grid(g.heads, n_tiles, NW == 8 ? 1 : 2);
   const int gate_off = g.heads * (g.dim + g.rot) + g.kr + g.rot;
-  hipLaunchKernelGGL((k_window_prefill<T, KS, DC, MR>), grid, dim3(256), lds,
+  hipLaunchKernelGGL((k_window_prefill<T, KS, DC, NW>), grid, dim3(NW * 64), lds,
                      stream, out, os, proj, ps, kv, krot, spans, tiles,
                      gate_off, g, vec);
 }

@@ -267,10 +267,10 @@ def latent_attn_decode(proj, out, m, w, rot, batch, rows,
     if m.window is not None:
         n_max = min(n_max, m.window)
     groups = B * -(-m.heads // 16)
-    splits = max(1, min(MAX_SPLITS, -(-n_max // 16),
+    splits = max(1, min(MAX_SPLITS, -(-n_max // 32),
                         -(-TARGET_BLOCKS // groups)))
     per_split = -(-n_max // splits)
-    tile = 16 if per_split <= 16 else 32 if per_split <= 32 else 64
+    tile = 32 if per_split <= 32 else 64
     qa = torch.empty(B, m.heads, m.row_width, dtype=proj.dtype, device=dev)
     part_o = torch.empty(B, m.heads, splits, m.kv_rank, dtype=torch.float32,
                          device=dev)
