@@ -71,6 +71,8 @@ def main(argv: Optional[List[str]] = None) -> int:
         req = json.loads(line)
         entries = []
         for e in req.get("entries", []):
+            if not e["tokens"]:
+                continue
             if e["id"] not in live:
                 live[e["id"]] = runner.admit()
             entries.append(StepEntry(live[e["id"]], e["tokens"],

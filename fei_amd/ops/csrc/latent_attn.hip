@@ -192,7 +192,7 @@ k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
   typedef typename El<T>::frag frag;
   constexpr int NP = Parts<T>::n;
   constexpr int NQ = 9;                    // steps per wave: R <= 4 * 9 * 32
-  constexpr int NL = 6;                    // row loads in flight per thread
+  constexpr int NL = 9;                    // row loads in flight per thread
   extern __shared__ __align__(16) char smem[];
   const int R = g.kr + g.rot;
   const int KP = (KT + 31) / 32 * 32;      // P columns, zero beyond KT
@@ -256,12 +256,14 @@ k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
     __syncthreads();
     if (vec) {
       const int nv = Rs / 8 - 1;           // vec8 slots that may be read
+      // i / nv for i < 2^16, as a product (nv > 1)
+      const unsigned per = 0xffffffffu / (unsigned)nv + 1u;
       for (int i0 = tid; i0 < KT * nv; i0 += 256 * NL) {
         frag v[NL];
 #pragma unroll
         for (int u = 0; u < NL; ++u) {
           const int i = i0 + u * 256;
-          const int r = i / nv, c = (i - r * nv) * 8;
+          const int r = __umulhi((unsigned)i, per), c = (i - r * nv) * 8;
 #pragma unroll
           for (int j = 0; j < 8; ++j) v[u][j] = 0;
           if (i < KT * nv && t0 + r < hi && c < R)
@@ -271,7 +273,7 @@ k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
 #pragma unroll
         for (int u = 0; u < NL; ++u) {
           const int i = i0 + u * 256;
-          const int r = i / nv, c = (i - r * nv) * 8;
+          const int r = __umulhi((unsigned)i, per), c = (i - r * nv) * 8;
           if (i < KT * nv) st8(ks + r * Rs + c, v[u]);
         }
       }

@@ -64,7 +64,7 @@ CONFIGS = {
                       (att(18, 24, 8, 40, 72, 64), 96)], width=64, vocab=96,
                      loop=(0, 2, 1), cap=None, scale=1.0),
     # attention without a window, one head, no loop
-    "full": make_cfg([(att(1, 32, 16, 48, 128, None), 40),
+    "full": make_cfg([(att(1, 40, 12, 56, 128, None), 40),
                       (lin(1, 64, 128, 8.0), 40)], width=48, vocab=77),
 }
 
@@ -261,6 +261,106 @@ def test_long_decoding(tmp_path, device):
     r = net.runner()
     got = run(r, r.admit(), tokens, [30] + [1] * 300)
     assert err(got, net.want(tokens)) < F32_TOL
+
+
+LARGE = {
+    # the sizes of a real model's layers
+    "usual": [att(16, 128, 64, 128, 512, 100), lin(4, 128, 256, 16.0)],
+    # the largest sizes the kernels take
+    "largest": [att(2, 192, 64, 256, 1024, 70), lin(2, 256, 512, 16.0)],
+    # between the sizes that kernels are built for, vector paths
+    "between": [att(5, 72, 24, 88, 136, 90), lin(3, 48, 104, 3.0)],
+    # the same without them
+    "ragged": [att(3, 67, 30, 85, 131, 90), lin(2, 45, 101, 3.0)],
+}
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("name", list(LARGE))
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_other_sizes(tmp_path, name, dtype):
+    cfg = make_cfg([(m, None) for m in LARGE[name]], width=64, vocab=40)
+    net = Net(tmp_path, cfg, 60, "cuda", dtype, gate_rank=16)
+    tokens = toks(140, 40, 61)
+    want = net.want(tokens)
+    r = net.runner(slots=1)
+    tol = F32_TOL if dtype == torch.float32 else 0.06
+    for sizes in ([140], [131, 1], [5, 66, 1]):
+        sid = r.admit()
+        assert err(run(r, sid, tokens, sizes), want) < tol, sizes
+        r.release(sid)
+
+
+# -- single ops on the GPU ----------------------------------------------------------
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("rows", [1, 2, 3, 4, 5, 8, 9, 33])
+@pytest.mark.parametrize("width,n_mix,ff", [(1024, 96, 64), (2048, 144, 2048),
+                                            (88, 30, 41), (52, 7, 0)])
+def test_products(rows, width, n_mix, ff):
+    """Every route of the skinny products against float64 on the same
+    bfloat16 values: rows per wave, shared K, matrix tile, library."""
+    g = torch.Generator().manual_seed(rows + width)
+    bf = lambda *s: torch.randn(*s, generator=g).bfloat16()
+    n1, n2 = bf(rows, width), bf(rows, width)
+    w_in = bf(n_mix + 2 * ff, width) / width ** 0.5
+    d = lambda t: t.double()
+    cat = torch.zeros(rows, n_mix + ff, dtype=torch.bfloat16, device="cuda")
+    proj = ops.mix_in(n1.cuda(), n2.cuda(), w_in.cuda(), n_mix, ff,
+                      cat[:, n_mix:])
+    assert err(proj, d(n1) @ d(w_in[:n_mix]).T) < 8e-3
+    if ff:
+        z = d(n2) @ d(w_in[n_mix:]).T
+        act = z[:, :ff] * torch.sigmoid(z[:, :ff]) * z[:, ff:]
+        assert err(cat[:, n_mix:], act) < 2e-2
+    w = bf(n_mix + 50, width) / width ** 0.5
+    x = torch.randn(rows, n_mix + 50, generator=g)
+    y = ops.residual_linear(x.cuda(), n1.cuda(), w.cuda())
+    assert err(y, d(x) + d(n1) @ d(w).T) < 1e-5
+    b = torch.randn(n_mix + 50, generator=g)
+    y = ops.linear_f32(n1.cuda(), w.cuda(), b.cuda())
+    assert err(y, d(n1) @ d(w).T + d(b)) < 1e-5
+    y = ops.logits_head(n1.cuda(), w.cuda(), 0.7, 2.0)
+    assert err(y, 2.0 * torch.tanh(d(n1) @ d(w).T * 0.35)) < 1e-5
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("cols", [64, 77])
+def test_row_ops(dtype, cols):
+    g = torch.Generator().manual_seed(cols)
+    x, y = (torch.randn(19, cols, generator=g) * 3 for _ in range(2))
+    w1, w2 = torch.randn(cols, generator=g), torch.randn(cols, generator=g)
+    tol = 1e-6 if dtype == torch.float32 else 4e-3
+    a, b = ops.norm_pair(x.cuda(), w1.cuda(), w2.cuda(), 1e-3, dtype)
+    want = oracle.rms(x.double(), 1e-3)
+    assert a.dtype == dtype
+    assert err(a, want * w1) < tol and err(b, want * w2) < tol
+    assert ops.norm_pair(x.cuda(), w1.cuda(), None, 1e-3, dtype)[1] is None
+    c = ops.cat_cast(x.cuda(), y.cuda(), dtype)
+    assert torch.equal(c.cpu(), torch.cat([x, y], 1).to(dtype))
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("batch", [3, 12])
+@pytest.mark.parametrize("vocab", [4096, 1003])
+def test_sampling_of_float32_logits(batch, vocab):
+    """Differences below bfloat16's resolution decide."""
+    g = torch.Generator().manual_seed(vocab)
+    logits = torch.rand(batch, vocab, generator=g)
+    best = torch.randint(0, vocab, (batch,), generator=g)
+    logits[torch.arange(batch), best] = 1.0001
+    logits[torch.arange(batch), (best + 1) % vocab] = 1.0
+    token = torch.zeros(batch, dtype=torch.int32, device="cuda")
+    step = torch.zeros(1, dtype=torch.int32, device="cuda")
+    ws = torch.zeros(batch, 128, device="cuda")
+    outs = torch.zeros(batch, 4, dtype=torch.int32, device="cuda")
+    ops.sample(logits.cuda(), token, step, ws, out_tokens=outs)
+    assert token.tolist() == best.tolist() == outs[:, 0].tolist()
+    ops.sample(logits.cuda() * 4, token, step, ws, temperature=0.8, seed=11)
+    noisy = logits * 5.0 + ops.ref.hash_gumbel(batch, vocab, 0, 11, 0)
+    for i, t in enumerate(token.tolist()):
+        assert float(noisy[i, t]) > float(noisy[i].max()) - 1e-3
 
 
 # -- window edges -------------------------------------------------------------------
