@@ -175,15 +175,16 @@ __device__ __forceinline__ T part_of(float v, int i) {
   return i == 0 ? hi : El<T>::st(v - El<T>::ld(hi));
 }
 
-// Decode partials. grid (splits, ceil(heads / 16), B), 4 waves. The visible
+// Decode partials. grid (splits, ceil(heads / 16 NH), B). The visible
 // keys of row b are cut into ``splits`` chunks of a multiple of KT keys; a
-// block walks its chunk in tiles of KT cached rows held in LDS. For the scores
-// the waves share out the 32-wide steps along a row (their sums meet in LDS),
-// for the weighted sum the columns.
+// block walks its chunk in tiles of KT cached rows held in LDS, which NH groups
+// of 4 waves use for 16 heads each. For the scores a group's waves share out
+// the 32-wide steps along a row (their sums meet in LDS), for the weighted sum
+// the columns.
 // NCT: 16-column tiles of the latent per wave (kr <= 64 * NCT).
 // part_o [B, H, splits, kr] unnormalised, part_ml [B, H, splits, 2].
-template <typename T, int NCT>
-__global__ void __launch_bounds__(256)
+template <typename T, int NCT, int NH>
+__global__ void __launch_bounds__(256 * NH)
 k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
                 float* __restrict__ part_o, float* __restrict__ part_ml,
                 const int* __restrict__ pos, const int* __restrict__ table,
@@ -192,29 +193,34 @@ k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
   typedef typename El<T>::frag frag;
   constexpr int NP = Parts<T>::n;
   constexpr int NQ = 9;                    // steps per wave: R <= 4 * 9 * 32
+  constexpr int NT = 256 * NH;
   constexpr int NL = 9;                    // row loads in flight per thread
   extern __shared__ __align__(16) char smem[];
   const int R = g.kr + g.rot;
   const int KP = (KT + 31) / 32 * 32;      // P columns, zero beyond KT
   const int KPs = KP + 8;
   T* ks = (T*)smem;                        // [KP][Rs]
-  T* ph = ks + KP * Rs;                    // [NP][16][KPs]
-  float* ss = (float*)(ph + NP * 16 * KPs);  // [4][16][KT + 1]
-  float* al = ss + 64 * (KT + 1);          // [16]
-
-  const int split = blockIdx.x, h0 = blockIdx.y * 16, b = blockIdx.z;
-  const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63;
+  const int split = blockIdx.x, b = blockIdx.z;
+  const int tid = threadIdx.x, grp = tid >> 8, w = (tid >> 6) & 3;
+  const int lane = tid & 63;
+  const int h0 = (blockIdx.y * NH + grp) * 16;
+  // per group: [NP][16][KPs], [4][16][KT + 1], [16]
+  T* ph = ks + KP * Rs + grp * NP * 16 * KPs;
+  float* ss = (float*)(ks + KP * Rs + NH * NP * 16 * KPs) +
+              grp * (64 * (KT + 1) + 16);
+  float* al = ss + 64 * (KT + 1);
   const int l15 = lane & 15, lg = lane >> 4;
   const int p = pos[b];
   const int k0 = first_key(p, g.window);
   const int n = p + 1 - k0;
   const int chunk = ((n + splits - 1) / splits + KT - 1) / KT * KT;
   const int lo = split * chunk, hi = min(lo + chunk, n);
-  const int nh = min(16, g.heads - h0);
+  const int nh = min(16, g.heads - h0);    // may be 0 or less in a last group
 
   if (lo >= hi) {
-    if (tid < nh) {
-      float* ml = part_ml + (((long)b * g.heads + h0 + tid) * splits + split) * 2;
+    const int h = tid & 255;
+    if (h < nh) {
+      float* ml = part_ml + (((long)b * g.heads + h0 + h) * splits + split) * 2;
       ml[0] = NEG_INF;
       ml[1] = 0.f;
     }
@@ -225,7 +231,7 @@ k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
   const int ksteps = (R + 31) / 32;
   frag q[NQ];
   {
-    const T* qr = qa + ((long)b * g.heads + h0 + min(l15, nh - 1)) * R;
+    const T* qr = qa + ((long)b * g.heads + h0 + max(min(l15, nh - 1), 0)) * R;
 #pragma unroll
     for (int i = 0; i < NQ; ++i) {
       const int k = w + 4 * i;
@@ -243,8 +249,8 @@ k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
       }
     }
   }
-  for (int i = tid; i < NP * 16 * KPs; i += 256) ph[i] = El<T>::st(0.f);
-  for (int i = KT * Rs + tid; i < KP * Rs; i += 256) ks[i] = El<T>::st(0.f);
+  for (int i = tid & 255; i < NP * 16 * KPs; i += 256) ph[i] = El<T>::st(0.f);
+  for (int i = KT * Rs + tid; i < KP * Rs; i += NT) ks[i] = El<T>::st(0.f);
 
   f32x4 acc[NCT];
 #pragma unroll
@@ -258,11 +264,11 @@ k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
       const int nv = Rs / 8 - 1;           // vec8 slots that may be read
       // i / nv for i < 2^16, as a product (nv > 1)
       const unsigned per = 0xffffffffu / (unsigned)nv + 1u;
-      for (int i0 = tid; i0 < KT * nv; i0 += 256 * NL) {
+      for (int i0 = tid; i0 < KT * nv; i0 += NT * NL) {
         frag v[NL];
 #pragma unroll
         for (int u = 0; u < NL; ++u) {
-          const int i = i0 + u * 256;
+          const int i = i0 + u * NT;
           const int r = __umulhi((unsigned)i, per), c = (i - r * nv) * 8;
 #pragma unroll
           for (int j = 0; j < 8; ++j) v[u][j] = 0;
@@ -272,13 +278,13 @@ k_latent_decode(const T* __restrict__ qa, const T* __restrict__ rows,
         }
 #pragma unroll
         for (int u = 0; u < NL; ++u) {
-          const int i = i0 + u * 256;
+          const int i = i0 + u * NT;
           const int r = __umulhi((unsigned)i, per), c = (i - r * nv) * 8;
           if (i < KT * nv) st8(ks + r * Rs + c, v[u]);
         }
       }
     } else {
-      for (int i = tid; i < KT * Rs; i += 256) {
+      for (int i = tid; i < KT * Rs; i += NT) {
         const int r = i / Rs, c = i - r * Rs;
         ks[i] = (t0 + r < hi && c < R)
                     ? rows[cache_row(table, W, b, k0 + t0 + r, bs_log) * R + c]
@@ -729,33 +735,39 @@ int run_decode(T* out, long os, const T* proj, long ps, const T* wuk,
                        bs_log, g, eps);
 
   const int Rs = (R + 31) / 32 * 32 + 8;
+  const int nh = g.heads > 16 ? 2 : 1;     // groups of 16 heads per block
   auto lds = [&](int KT) {
     const int KP = (KT + 31) / 32 * 32;
-    return (size_t)sizeof(T) * (KP * Rs + Parts<T>::n * 16 * (KP + 8)) +
-           4 * (64 * (KT + 1) + 16);
+    return (size_t)sizeof(T) * (KP * Rs + nh * Parts<T>::n * 16 * (KP + 8)) +
+           4 * nh * (64 * (KT + 1) + 16);
   };
   int KT = tile;
   while (KT > 16 && lds(KT) > 160 * 1024) KT >>= 1;
   if (lds(KT) > 160 * 1024 || R > 1152) return 1;
-  const dim3 gd(splits, (g.heads + 15) / 16, B);
-#define DEC(N)                                                               \
+  const dim3 gd(splits, (g.heads + 16 * nh - 1) / (16 * nh), B);
+#define DEC(N, H)                                                            \
   do {                                                                       \
     static bool set = false;                                                 \
     if (!set) {                                                              \
-      (void)hipFuncSetAttribute((const void*)k_latent_decode<T, N>,          \
+      (void)hipFuncSetAttribute((const void*)k_latent_decode<T, N, H>,       \
                                 hipFuncAttributeMaxDynamicSharedMemorySize,  \
                                 160 * 1024);                                 \
       set = true;                                                            \
     }                                                                        \
-    hipLaunchKernelGGL((k_latent_decode<T, N>), gd, dim3(256), lds(KT),      \
-                       stream, qa, rows, part_o, part_ml, pos, table, W,     \
-                       bs_log, g, splits, KT, Rs, R % 8 == 0);               \
+    hipLaunchKernelGGL((k_latent_decode<T, N, H>), gd, dim3(256 * H),        \
+                       lds(KT), stream, qa, rows, part_o, part_ml, pos,      \
+                       table, W, bs_log, g, splits, KT, Rs, R % 8 == 0);     \
+  } while (0)
+#define BY_NCT(H)               \
+  do {                          \
+    if (nct <= 2) DEC(2, H);    \
+    else if (nct <= 4) DEC(4, H); \
+    else if (nct <= 8) DEC(8, H); \
+    else DEC(16, H);            \
   } while (0)
   const int nct = (g.kr + 63) / 64;
-  if (nct <= 2) DEC(2);
-  else if (nct <= 4) DEC(4);
-  else if (nct <= 8) DEC(8);
-  else DEC(16);
+  if (nh == 2) BY_NCT(2); else BY_NCT(1);
+#undef BY_NCT
 #undef DEC
 
   const dim3 go(g.heads, (g.vdim + 15) / 16, B);

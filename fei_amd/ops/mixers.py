@@ -266,11 +266,11 @@ def latent_attn_decode(proj, out, m, w, rot, batch, rows,
     n_max = W * block_size
     if m.window is not None:
         n_max = min(n_max, m.window)
-    groups = B * -(-m.heads // 16)
+    groups = B * -(-m.heads // 32)
     splits = max(1, min(MAX_SPLITS, -(-n_max // 32),
                         -(-TARGET_BLOCKS // groups)))
     per_split = -(-n_max // splits)
-    tile = 32 if per_split <= 32 else 64
+    tile = 32 if per_split <= 48 else 64
     qa = torch.empty(B, m.heads, m.row_width, dtype=proj.dtype, device=dev)
     part_o = torch.empty(B, m.heads, splits, m.kv_rank, dtype=torch.float32,
                          device=dev)
