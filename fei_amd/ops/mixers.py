@@ -8,7 +8,6 @@ the dtype of the rows; CPU tensors to the reference implementations.
 from __future__ import annotations
 
 import ctypes
-import os
 from typing import Optional, Tuple
 
 import torch
