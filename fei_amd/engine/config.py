@@ -1,9 +1,11 @@
 """Model specs for the local engine.
 
-Two families of decoder: ``ModelSpec`` (one attention layer repeated;
-Llama-3) and ``TobaraxSpec`` (a list of unlike layers, each with its own
-mixer and sizes, part of the list run several times in a row). ``get_spec``
-takes a registered name or a folder with a config.json.
+Three families of decoder: ``ModelSpec`` (one attention layer repeated;
+Llama-3), ``TobaraxSpec`` (a list of unlike layers, each with its own mixer
+and sizes, part of the list run several times in a row) and ``BokenexSpec`` (a
+list of parallel layers: sigmoid attention beside a dense feed-forward or a
+mixture of experts). ``get_spec`` takes a registered name or a folder with a
+config.json.
 
 Llama-3 8B/70B shapes per the BASELINE.json configs (weights are random-init
 — there is no network for checkpoints; bench.py states data=synthetic).
@@ -34,6 +36,8 @@ class ModelSpec:
     norm_eps: float = 1e-5
     max_seq_len: int = 8192
     arch: str = "llama"           # "llama" (decoder) | "bert" (encoder)
+
+    max_positions = None          # positions past which it cannot go
 
     @property
     def q_size(self) -> int:
@@ -118,7 +122,65 @@ class GLASpec:
         return self.heads * self.dim * self.vdim
 
 
-MixerSpec = Union[LatentAttentionSpec, GLASpec]
+@dataclass(frozen=True)
+class SigmoidAttentionSpec:
+    """Grouped-query attention whose key weights are sigmoids, not a softmax.
+
+    q, k and v pass a causal convolution of ``conv`` taps per channel; q and k
+    an RMS norm per head. A score is scale * (q . k) - r1 ln(1 + r2 d) at
+    distance d, a weight sigmoid(score + pb), with r1, r2, pb per head.
+    ``window``: a query sees that many positions, itself included (None =
+    all)."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    conv: int = 1
+    window: Optional[int] = None
+
+    kind = "attention"
+
+    @property
+    def in_rows(self) -> int:
+        """Rows of the stacked q, k, v projections."""
+        return self.heads * self.dim + self.row_width
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def row_width(self) -> int:
+        """Cached values per token: keys, then values, of every kv head."""
+        return self.kv_heads * (self.dim + self.vdim)
+
+
+MixerSpec = Union[LatentAttentionSpec, GLASpec, SigmoidAttentionSpec]
+
+
+@dataclass(frozen=True)
+class DenseSpec:
+    """W_down relu(W_up h)^2."""
+    ff: int
+
+    kind = "dense"
+
+
+@dataclass(frozen=True)
+class MoESpec:
+    """``top`` of ``experts`` feed-forwards of width ``ff`` per token, by
+    sigmoid router scores; their weights are the chosen scores over their sum,
+    times ``scale``."""
+    experts: int
+    top: int
+    ff: int
+    scale: float = 1.0
+
+    kind = "moe"
+
+
+MlpSpec = Union[DenseSpec, MoESpec]
 
 
 @dataclass(frozen=True)
@@ -159,6 +221,8 @@ class TobaraxSpec:
     loop: Optional[LoopSpec] = None
     max_seq_len: int = 8192
     arch: str = "tobarax"
+
+    max_positions = None          # rotations have no last position
 
     def __post_init__(self) -> None:
         if self.loop is not None:
@@ -291,7 +355,137 @@ class TobaraxSpec:
         return out
 
 
-AnySpec = Union[ModelSpec, TobaraxSpec]
+@dataclass(frozen=True)
+class ParallelLayerSpec:
+    """Mixer and feed-forward read the same normed input."""
+    mixer: SigmoidAttentionSpec
+    mlp: Optional[MlpSpec] = None
+
+
+@dataclass(frozen=True)
+class BokenexSpec:
+    """``max_seq_len`` is the number of learned position vectors."""
+    name: str
+    vocab_size: int
+    hidden_size: int
+    layers: Tuple[ParallelLayerSpec, ...]
+    norm_eps: float
+    residual_mult: float
+    max_seq_len: int
+    arch: str = "bokenex"
+
+    @property
+    def max_positions(self) -> Optional[int]:
+        """Positions past which the model cannot go."""
+        return self.max_seq_len
+
+    def __post_init__(self) -> None:
+        for i, L in enumerate(self.layers):
+            m = L.mixer
+            if min(m.heads, m.kv_heads, m.dim, m.vdim, m.conv) < 1 \
+                    or m.heads % m.kv_heads \
+                    or (m.window is not None and m.window < 1):
+                raise ValueError(f"layer {i}: impossible mixer {m}")
+            if L.mlp is not None and L.mlp.kind == "moe" and \
+                    not 1 <= L.mlp.top <= L.mlp.experts:
+                raise ValueError(f"layer {i}: {L.mlp.top} of "
+                                 f"{L.mlp.experts} experts")
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def intermediate_size(self) -> int:
+        """Widest feed-forward, all experts of a layer together."""
+        return max((L.mlp.ff * getattr(L.mlp, "experts", 1)
+                    for L in self.layers if L.mlp is not None), default=0)
+
+    def params_bytes(self, dtype_bytes: int = 2) -> int:
+        C = self.hidden_size
+        total = (2 * self.vocab_size + self.max_seq_len) * C + 1
+        for L in self.layers:
+            m = L.mixer
+            total += (C + m.conv) * m.in_rows + C * m.out_cols
+            total += 2 * m.dim + 3 * m.heads + 1
+            if L.mlp is not None and L.mlp.kind == "moe":
+                total += L.mlp.experts * C * (1 + 2 * L.mlp.ff)
+            elif L.mlp is not None:
+                total += 2 * C * L.mlp.ff
+        return total * dtype_bytes
+
+    # -- config.json -----------------------------------------------------------
+
+    @classmethod
+    def from_config(cls, cfg: Dict[str, Any], shapes: Dict[str, Tuple[int, ...]],
+                    name: str = "bokenex") -> "BokenexSpec":
+        """Keys that this class does not know are refused rather than
+        skipped. ``shapes`` is not needed: the configuration has all sizes."""
+        _only(cfg, ("architecture", "layers", "max_positions", "norm",
+                    "residual_mult", "vocab", "width"), "config")
+        layers = []
+        for i, L in enumerate(cfg["layers"]):
+            where = f"layer {i}"
+            _only(L, ("type", "mixer", "mlp"), where)
+            if L["type"] != "attention":
+                raise ValueError(f"{where}: unknown type {L['type']!r}")
+            m, mask = L["mixer"], L["mixer"].get("mask") or {}
+            _only(m, ("conv", "dim", "heads", "kv_heads", "mask", "scale",
+                      "vdim"), where)
+            _only(mask, ("size",), where)
+            mixer = SigmoidAttentionSpec(
+                heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"],
+                vdim=m["vdim"], scale=float(m["scale"]), conv=m["conv"],
+                window=mask.get("size"))
+            layers.append(ParallelLayerSpec(
+                mixer, _mlp(L["mlp"], where) if L.get("mlp") else None))
+        return cls(
+            name=name, vocab_size=cfg["vocab"], hidden_size=cfg["width"],
+            layers=tuple(layers), norm_eps=float(cfg["norm"]["eps"]),
+            residual_mult=float(cfg["residual_mult"]),
+            max_seq_len=int(cfg["max_positions"]))
+
+    def to_config(self) -> Dict[str, Any]:
+        layers = []
+        for L in self.layers:
+            m, f = L.mixer, L.mlp
+            mixer = {"heads": m.heads, "kv_heads": m.kv_heads, "dim": m.dim,
+                     "vdim": m.vdim, "scale": m.scale, "conv": m.conv}
+            if m.window is not None:
+                mixer["mask"] = {"size": m.window}
+            mlp = None
+            if f is not None and f.kind == "moe":
+                mlp = {"kind": "moe", "expert": {"ff": f.ff},
+                       "router": {"experts": f.experts, "top": f.top,
+                                  "scale": f.scale}}
+            elif f is not None:
+                mlp = {"kind": "dense", "ff": f.ff}
+            layers.append({"type": m.kind, "mixer": mixer, "mlp": mlp})
+        return {"architecture": "Bokenex", "layers": layers,
+                "max_positions": self.max_seq_len,
+                "norm": {"eps": self.norm_eps},
+                "residual_mult": self.residual_mult,
+                "vocab": self.vocab_size, "width": self.hidden_size}
+
+
+def _mlp(f: Dict[str, Any], where: str) -> MlpSpec:
+    if f["kind"] == "dense":
+        _only(f, ("kind", "ff"), where)
+        return DenseSpec(int(f["ff"]))
+    if f["kind"] != "moe":
+        raise ValueError(f"{where}: unknown mlp {f['kind']!r}")
+    r = f["router"]
+    _only(f, ("kind", "expert", "router"), where)
+    _only(f["expert"], ("ff",), where)
+    _only(r, ("experts", "top", "scale"), where)
+    return MoESpec(experts=int(r["experts"]), top=int(r["top"]),
+                   ff=int(f["expert"]["ff"]), scale=float(r["scale"]))
+
+
+AnySpec = Union[ModelSpec, TobaraxSpec, BokenexSpec]
+
+# config.json's "architecture" -> spec
+ARCHITECTURES = {"Tobarax": TobaraxSpec, "Bokenex": BokenexSpec}
 
 
 def _tobarax(name: str, vocab: int, width: int, ff: int, heads: int,
@@ -310,6 +504,22 @@ def _tobarax(name: str, vocab: int, width: int, ff: int, heads: int,
         layers=tuple(LayerSpec(att if c == "a" else gla, ff) for c in pattern),
         norm_eps=1e-5, logit_scale=0.5, logit_softcap=30.0, loop=loop,
         max_seq_len=max_seq_len)
+
+
+def _bokenex(name: str, vocab: int, width: int, heads: int, kv_heads: int,
+             dim: int, vdim: int, window: int, pattern: str, dense: DenseSpec,
+             moe: MoESpec, conv: int = 4,
+             max_seq_len: int = 8192) -> BokenexSpec:
+    """``pattern``: one letter per layer, 'd' dense, 'm' mixture of experts,
+    '-' without a feed-forward."""
+    att = SigmoidAttentionSpec(heads=heads, kv_heads=kv_heads, dim=dim,
+                               vdim=vdim, scale=dim ** -0.5, conv=conv,
+                               window=window)
+    mlp = {"d": dense, "m": moe, "-": None}
+    return BokenexSpec(
+        name=name, vocab_size=vocab, hidden_size=width,
+        layers=tuple(ParallelLayerSpec(att, mlp[c]) for c in pattern),
+        norm_eps=1e-5, residual_mult=0.5, max_seq_len=max_seq_len)
 
 
 MODEL_SPECS: Dict[str, AnySpec] = {
@@ -362,6 +572,22 @@ MODEL_SPECS: Dict[str, AnySpec] = {
         pattern="ag" * 15, loop=LoopSpec(14, 16, 2), dim=128, rot=64,
         vdim=128, kv_rank=512, window=4096, gla_heads=16, gla_dim=128,
         gla_vdim=256),
+    # Bokenex: layers of sigmoid attention beside a dense feed-forward or a
+    # mixture of experts. The 1b/8b shapes have the width, heads and
+    # vocabulary of the llama3 specs beside them, and feed-forwards of as many
+    # parameters.
+    "bokenex-tiny": _bokenex(
+        "bokenex-tiny", vocab=304, width=80, heads=4, kv_heads=2, dim=24,
+        vdim=40, window=40, pattern="dm-m", dense=DenseSpec(112),
+        moe=MoESpec(6, 2, 48, 1.25), conv=3, max_seq_len=512),
+    "bokenex-1b": _bokenex(
+        "bokenex-1b", vocab=128256, width=2048, heads=32, kv_heads=8, dim=64,
+        vdim=64, window=1024, pattern="dm" * 8, dense=DenseSpec(12288),
+        moe=MoESpec(16, 4, 768, 1.5)),
+    "bokenex-8b": _bokenex(
+        "bokenex-8b", vocab=128256, width=4096, heads=32, kv_heads=8, dim=128,
+        vdim=128, window=4096, pattern="dm" * 16, dense=DenseSpec(21504),
+        moe=MoESpec(16, 4, 1344, 1.5)),
 }
 
 
@@ -383,12 +609,13 @@ def load_spec(path: str) -> AnySpec:
     if "arch" in cfg:                      # written by LlamaModel.save_weights
         known = {f.name for f in fields(ModelSpec)}
         return ModelSpec(**{k: v for k, v in cfg.items() if k in known})
-    if cfg.get("architecture") == "Tobarax":
-        shapes = tensor_shapes(os.path.join(path, "model.safetensors"))
-        return TobaraxSpec.from_config(
-            cfg, shapes, name=os.path.basename(os.path.abspath(path)))
-    raise ValueError(f"{path}: unknown architecture "
-                     f"{cfg.get('architecture')!r}")
+    cls = ARCHITECTURES.get(cfg.get("architecture"))
+    if cls is None:
+        raise ValueError(f"{path}: unknown architecture "
+                         f"{cfg.get('architecture')!r}")
+    shapes = tensor_shapes(os.path.join(path, "model.safetensors"))
+    return cls.from_config(cfg, shapes,
+                           name=os.path.basename(os.path.abspath(path)))
 
 
 def is_model_folder(name: str) -> bool:

@@ -311,7 +311,7 @@ class LocalEngine:
         per_tok = self._kv_bytes_per_token() * self.B
         seq = min(budget // per_tok, 262144)
         seq = max((seq // 1024) * 1024, self.spec.max_seq_len)
-        return int(seq)
+        return int(min(seq, self.spec.max_positions or seq))
 
     @classmethod
     def create(cls, model: Union[str, AnySpec] = "llama3-8b", **kwargs) -> "LocalEngine":

@@ -50,6 +50,16 @@ class RaggedBatch:
         t = torch.from_numpy(np.asarray(rows, dtype=np.int32))
         return t.view(-1, width).to(self.tokens.device)
 
+    def span_plan(self):
+        """The prompt portions [first row, rows, first position], and their
+        query tiles [portion, first row in it]."""
+        if "spans" not in self._plans:
+            tiles = [[p, q] for p, (_, n, _) in enumerate(self.portions)
+                     for q in range(0, n, Q_TILE)]
+            self._plans["spans"] = (self._upload(self.portions, 3),
+                                    self._upload(tiles, 2))
+        return self._plans["spans"]
+
     def key_plan(self, window: Optional[int]):
         """What the prompt portions read through a window: per portion
         [first row, rows, first position, first key position, first packed

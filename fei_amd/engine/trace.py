@@ -59,8 +59,9 @@ def main(argv: Optional[List[str]] = None) -> int:
               file=sys.stderr)
         return 2
     blocks = -(-args.max_tokens // BLOCK)
+    longest = min(blocks * BLOCK, spec.max_positions or blocks * BLOCK)
     model = cls(spec, device, getattr(torch, args.dtype),
-                max_seq_len=blocks * BLOCK, weights=args.model)
+                max_seq_len=longest, weights=args.model)
     runner = StepRunner(model, num_blocks=blocks, num_slots=SLOTS,
                         block_size=BLOCK)
 

@@ -1,9 +1,11 @@
 """Model classes by architecture."""
 
+from fei_amd.models.bokenex import BokenexModel
 from fei_amd.models.llama import LlamaModel
 from fei_amd.models.tobarax import TobaraxModel
 
-MODEL_CLASSES = {"llama": LlamaModel, "tobarax": TobaraxModel}
+MODEL_CLASSES = {"llama": LlamaModel, "tobarax": TobaraxModel,
+                 "bokenex": BokenexModel}
 
 
 def model_class(spec):
@@ -15,4 +17,4 @@ def model_class(spec):
                          f"{spec.arch!r}") from None
 
 
-__all__ = ["LlamaModel", "MODEL_CLASSES", "TobaraxModel", "model_class"]
+__all__ = ["BokenexModel", "LlamaModel", "MODEL_CLASSES", "TobaraxModel", "model_class"]

@@ -12,7 +12,8 @@ from typing import Callable, Dict, Optional, Tuple
 import torch
 
 from fei_amd import ops
-from fei_amd.engine.config import GLASpec, LatentAttentionSpec
+from fei_amd.engine.config import (GLASpec, LatentAttentionSpec,
+                                   SigmoidAttentionSpec)
 
 Get = Callable[[str], torch.Tensor]
 
@@ -112,4 +113,54 @@ class GatedLinearAttention(Mixer):
             ops.gla_prefill(proj, out, *args)
 
 
-MIXERS = {"latent_attention": LatentAttention, "gla": GatedLinearAttention}
+class SigmoidAttention(Mixer):
+    """Grouped-query attention with sigmoid key weights, a logarithmic
+    distance bias and a sliding window, behind a short convolution over time
+    and query/key norms. A cached row is the normed keys and the values; the
+    state is the last ``conv`` projections, that of position p at p % conv."""
+
+    IN = ("q", "k", "v")
+
+    @staticmethod
+    def shapes(m: SigmoidAttentionSpec, width: int) -> Dict[str, tuple]:
+        nq, nk, nv = m.heads * m.dim, m.kv_heads * m.dim, m.kv_heads * m.vdim
+        return {"q": (nq, width), "k": (nk, width), "v": (nv, width),
+                "q.conv": (nq, m.conv), "k.conv": (nk, m.conv),
+                "v.conv": (nv, m.conv), "q.norm": (m.dim,),
+                "k.norm": (m.dim,), "r1": (m.heads,), "r2": (m.heads,),
+                "pb": (m.heads,), "o": (width, m.heads * m.vdim)}
+
+    def __init__(self, m: SigmoidAttentionSpec, eps: float, mat: Get,
+                 vec: Get):
+        ops.check_sigmoid_geometry(m)
+        self.m, self.eps = m, eps
+        self.qn, self.kn = vec("q.norm"), vec("k.norm")
+        # per head: r1, r2, pb
+        self.bias = torch.stack([vec("r1"), vec("r2"), vec("pb")]).contiguous()
+        # tap-major, so that the channels of a tap are contiguous
+        self.conv = torch.cat([vec(n + ".conv") for n in self.IN]).t() \
+            .contiguous()
+        self.row_width = m.row_width
+        if m.conv > 1:
+            self.state_shape = (m.conv, m.in_rows)
+
+    def own_weights(self) -> Dict[str, torch.Tensor]:
+        m = self.m
+        cq, ck, cv = self.conv.t().split(
+            [m.heads * m.dim, m.kv_heads * m.dim, m.kv_heads * m.vdim])
+        return {"q.norm": self.qn, "k.norm": self.kn, "r1": self.bias[0],
+                "r2": self.bias[1], "pb": self.bias[2], "q.conv": cq,
+                "k.conv": ck, "v.conv": cv}
+
+    def run(self, proj, out, batch, cache, run, rot) -> None:
+        args = (self.m, self, batch, cache.rows[run], cache.states[run],
+                cache.block_size)
+        n = batch.n_dec
+        if n:
+            ops.sigmoid_attn_decode(proj[:n], out[:n], *args)
+        if batch.portions:
+            ops.sigmoid_attn_prefill(proj, out, *args)
+
+
+MIXERS = {"latent_attention": LatentAttention, "gla": GatedLinearAttention,
+          "attention": SigmoidAttention}

@@ -6,17 +6,11 @@ both norms, one stacked product makes all projections of the layer, and one
 product over the concatenated outputs adds to the residual). Part of the
 layer list runs several times with the same weights; a pass begins with a
 linear map of the residual and the embedding, and adds a vector of its own.
-
-``forward`` runs one RaggedBatch (engine/step.py): prompts, portions of them
-and decoding sequences, in any mixture. With single tokens only, nothing in it
-depends on host values, so the step can be captured into a hipGraph.
 """
 
 from __future__ import annotations
 
-import json
 import math
-import os
 from dataclasses import dataclass
 from typing import Callable, Dict, List, Optional
 
@@ -26,8 +20,8 @@ from fei_amd import ops
 from fei_amd.engine.config import TobaraxSpec
 from fei_amd.engine.kv_cache import HybridCache
 from fei_amd.models.mixers import MIXERS, Mixer
+from fei_amd.models.step_model import StepModel
 from fei_amd.ops import reference as ref
-from fei_amd.parallel.pg import ParallelContext
 
 
 @dataclass
@@ -39,31 +33,13 @@ class TobaraxLayer:
     mixer: Mixer
 
 
-class TobaraxModel:
-    step_cache = True                   # runs RaggedBatches over a HybridCache
+class TobaraxModel(StepModel):
 
-    def __init__(self, spec: TobaraxSpec, device: torch.device,
-                 dtype: torch.dtype = torch.bfloat16,
-                 tp: Optional[ParallelContext] = None, seed: int = 1234,
-                 max_seq_len: Optional[int] = None,
-                 weights: Optional[str] = None):
-        if tp is not None and tp.is_distributed:
-            raise ValueError(f"{spec.name}: tensor parallelism is not "
-                             "available for this architecture")
-        self.spec = spec
-        self.device = torch.device(device)
-        self.dtype = dtype
-        self.tp = tp or ParallelContext()
-        self.tp_size = 1
-        # a decay carries every earlier token: the state cannot go back
-        self.recurrent = any(L.mixer.kind == "gla" for L in spec.layers)
-        self._set_weights(self._read(weights) if weights
-                          else self._random(seed))
-        self.resize(max_seq_len or spec.max_seq_len)
+    def mixers(self) -> List[Mixer]:
+        return [self.layers[r.layer].mixer for r in self.spec.runs]
 
     def resize(self, max_seq_len: int) -> None:
-        """Positions up to ``max_seq_len`` - 1 can be run from now on."""
-        self.max_seq_len = max_seq_len
+        super().resize(max_seq_len)
         keys = {(L.mixer.rot_dim, L.mixer.rot_base) for L in self.spec.layers
                 if L.mixer.kind == "latent_attention"}
         self._rot = {k: ref.rope_table_exact(max_seq_len, *k,
@@ -111,27 +87,6 @@ class TobaraxModel:
             return t * scale
         return get
 
-    def _read(self, path: str) -> Callable[[str], torch.Tensor]:
-        """Tensors of a model folder, one at a time; names and shapes have to
-        be exactly those of the spec."""
-        from safetensors import safe_open
-
-        f = safe_open(os.path.join(path, "model.safetensors"), framework="pt")
-        shapes = self._shapes()
-        names = set(f.keys())
-        if names != set(shapes):
-            raise ValueError(
-                f"{path}: missing tensors {sorted(set(shapes) - names)[:4]}, "
-                f"unknown tensors {sorted(names - set(shapes))[:4]}")
-
-        def get(name: str) -> torch.Tensor:
-            t = f.get_tensor(name)
-            if tuple(t.shape) != tuple(shapes[name]):
-                raise ValueError(f"{path}: {name} has shape {tuple(t.shape)},"
-                                 f" expected {tuple(shapes[name])}")
-            return t.to(self.device)
-        return get
-
     def _set_weights(self, get: Callable[[str], torch.Tensor]) -> None:
         s, dt = self.spec, self.dtype
         mat = lambda name: get(name).to(dt).contiguous()
@@ -159,11 +114,7 @@ class TobaraxModel:
         self.loop_in = mat("loop.in") if s.loop is not None else None
         self.loop_step = vec("loop.step") if s.loop is not None else None
 
-    def load_weights(self, path: str) -> None:
-        self._set_weights(self._read(path))
-
     def state_dict_full(self) -> Dict[str, torch.Tensor]:
-        """Tensors under their names in a model folder."""
         s, out = self.spec, {"embed": self.emb, "head": self.lm_head,
                              "final.norm": self.norm_f}
         if s.loop is not None:
@@ -185,36 +136,6 @@ class TobaraxModel:
                 out[p + "mlp.up"] = lw.w_in[at + L.ff:]
                 out[p + "mlp.down"] = lw.w_out[:, m.out_cols:]
         return out
-
-    def save_weights(self, path: str) -> None:
-        """Write a model folder (bfloat16, as such folders are)."""
-        from safetensors.torch import save_file
-
-        os.makedirs(path, exist_ok=True)
-        save_file({k: v.to(torch.bfloat16).contiguous().cpu()
-                   for k, v in self.state_dict_full().items()},
-                  os.path.join(path, "model.safetensors"))
-        with open(os.path.join(path, "config.json"), "w",
-                  encoding="utf-8") as f:
-            json.dump(self.spec.to_config(), f, indent=1)
-
-    def param_bytes(self) -> int:
-        return sum(t.numel() * t.element_size()
-                   for t in self.state_dict_full().values())
-
-    # -- cache -----------------------------------------------------------------
-
-    def new_cache(self, num_blocks: int, num_slots: int,
-                  block_size: int = 64) -> HybridCache:
-        mixers = [self.layers[r.layer].mixer for r in self.spec.runs]
-        return HybridCache(
-            [m.row_width for m in mixers], [m.state_shape for m in mixers],
-            num_blocks, num_slots, block_size, self.device, self.dtype)
-
-    def cache_bytes_per_token(self) -> int:
-        el = torch.empty(0, dtype=self.dtype).element_size()
-        return el * sum(self.layers[r.layer].mixer.row_width or 0
-                        for r in self.spec.runs)
 
     # -- forward -----------------------------------------------------------------
 

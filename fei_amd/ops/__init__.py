@@ -20,11 +20,18 @@ from typing import Optional, Tuple
 import torch
 
 from fei_amd.ops import mixers as _mixers
+from fei_amd.ops import moe as _moe
 from fei_amd.ops import reference as ref
+from fei_amd.ops import sigmoid_attn as _sigmoid_attn
 from fei_amd.ops.mixers import (  # noqa: F401
-    cat_cast, check_gla_geometry, check_latent_geometry, gla_decode,
-    gla_prefill, latent_attn_decode, latent_attn_prefill, linear_f32,
-    logits_head, mix_in, norm_pair, residual_linear)
+    GainNorm, GainNormed, cat_cast, check_gla_geometry,
+    check_latent_geometry, embed_pos, gain_logits, gla_decode, gla_prefill,
+    latent_attn_decode, latent_attn_prefill, linear_f32, logits_head, mix_in,
+    norm_pair, parallel_in, residual_linear)
+from fei_amd.ops.moe import (  # noqa: F401
+    check_moe_geometry, residual_moe, route)
+from fei_amd.ops.sigmoid_attn import (  # noqa: F401
+    check_sigmoid_geometry, sigmoid_attn_decode, sigmoid_attn_prefill)
 
 _LIB: Optional[ctypes.CDLL] = None
 _LIB_ERR: Optional[str] = None
@@ -95,6 +102,8 @@ def _try_load() -> None:
     lib.fei_gemv_swiglu_norm.argtypes = [_vp, _vp, _vp, _vp, _i, _i, _i, _f,
                                          _i, _vp, _vp]
     _mixers.declare(lib)
+    _moe.declare(lib)
+    _sigmoid_attn.declare(lib)
     _LIB = lib
 
 

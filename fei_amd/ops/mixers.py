@@ -1,4 +1,5 @@
-"""Ops of decoders made of unlike layers (models/tobarax.py, models/mixers.py).
+"""Ops of decoders made of unlike layers (models/tobarax.py, models/bokenex.py,
+models/mixers.py).
 
 Same dispatch rule as the rest of ``fei_amd.ops``: GPU tensors go to the HIP
 kernels (csrc/hybrid.hip, latent_attn.hip, gla.hip), in bfloat16 or float32 by
@@ -28,6 +29,13 @@ def declare(lib: ctypes.CDLL) -> None:
     lib.fei_softcap.argtypes = [_vp, _l, _f, _f, _vp]
     lib.fei_gemv_mix_in.argtypes = [_vp] * 5 + [_l] + [_i] * 4 + [_i, _vp]
     lib.fei_gemv_f32.argtypes = [_vp] * 4 + [_i] * 3 + [_i, _f, _f, _i, _vp]
+    lib.fei_embed_pos.argtypes = [_vp] * 5 + [_i] * 3 + [_vp]
+    lib.fei_relu2_rows.argtypes = [_vp, _l, _vp, _l, _i, _i, _i, _vp]
+    lib.fei_gemv_gain.argtypes = [_vp] * 4 + [_f] + [_i] * 3 + [_vp]
+    lib.fei_gemv_parallel_in.argtypes = (
+        [_vp] * 5 + [_f] + [_vp, _l] + [_i] * 5 + [_vp])
+    lib.fei_gemm_m8_parallel_in.argtypes = (
+        [_vp] * 5 + [_l] + [_i] * 5 + [_vp])
     lib.fei_gemm_m8_f32.argtypes = [_vp] * 4 + [_i] * 4 + [_f, _f, _vp]
     lib.fei_latent_decode.argtypes = (
         [_vp, _l, _vp, _l] + [_vp] * 10 + [_i] * 8 +
@@ -99,6 +107,56 @@ def cat_cast(x: torch.Tensor, y: torch.Tensor,
     return out
 
 
+def embed_pos(tokens: torch.Tensor, pos: torch.Tensor, emb: torch.Tensor,
+              pos_emb: torch.Tensor) -> torch.Tensor:
+    """emb[tokens] + pos_emb[pos], float32 [T, C]."""
+    if not emb.is_cuda:
+        return emb[tokens.long()].float() + pos_emb[pos.long()].float()
+    T, C = tokens.shape[0], emb.shape[1]
+    out = torch.empty(T, C, dtype=torch.float32, device=emb.device)
+    if tokens.dtype not in (torch.int32, torch.int64):
+        raise TypeError(f"token ids are {tokens.dtype}")
+    if T:
+        _lib().fei_embed_pos(
+            _p(out), _p(tokens.contiguous()), _p(pos), _p(emb), _p(pos_emb),
+            T, C, _f32(emb) | (2 if tokens.dtype == torch.int64 else 0),
+            _stream())
+    return out
+
+
+class GainNorm:
+    """RMS norm with one gain for all columns."""
+
+    def __init__(self, gain: torch.Tensor, width: int, eps: float):
+        self.gain, self.eps = gain, eps
+        # as a weight per column, for the norm of rows
+        self.cols = gain.expand(width).contiguous()
+
+
+class GainNormed:
+    """Rows x (float32) under a GainNorm. The gain and the root mean square
+    commute with a product, so a product of a row or two takes x as it is
+    and makes the norm inside; the others take the normed ``rows``."""
+
+    def __init__(self, x: torch.Tensor, norm: GainNorm, dtype: torch.dtype):
+        self.x, self.norm, self.dtype = x, norm, dtype
+        self._rows: Optional[torch.Tensor] = None
+
+    @property
+    def rows(self) -> torch.Tensor:
+        if self._rows is None:
+            self._rows, _ = norm_pair(self.x, self.norm.cols, None,
+                                      self.norm.eps, self.dtype)
+        return self._rows
+
+    @property
+    def inside(self) -> bool:
+        """Whether products make the norm inside."""
+        return (self.x.is_cuda and self.dtype == torch.bfloat16
+                and self.x.shape[0] <= 2 and self.x.shape[1] % 8 == 0
+                and self.x.shape[0] > 0)
+
+
 def _gemv_rows(T: int, K: int, t: torch.Tensor) -> bool:
     return T in (1, 2, 4, 8) and K % 8 == 0 and t.dtype == torch.bfloat16
 
@@ -144,6 +202,56 @@ def mix_in(n1: torch.Tensor, n2: Optional[torch.Tensor], w_in: torch.Tensor,
     return proj
 
 
+def parallel_in(h: GainNormed, w_in: torch.Tensor, n_mix: int, ff: int,
+                n_router: int, act: torch.Tensor
+                ) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
+    """All products of a parallel layer's input. The rows of ``w_in`` are
+    n_mix of the mixer, whose products are returned, then either ``ff`` of a
+    feed-forward, relu(.)^2 of which goes into ``act`` (a column range of a
+    wider buffer), or ``n_router`` of a router, whose float32 logits are
+    returned second (None without)."""
+    x, norm = h.x, h.norm
+    T, K = x.shape
+    n = n_mix + ff + n_router
+    gpu = x.is_cuda and h.dtype == torch.bfloat16
+    if h.inside or (gpu and _m8(T, K, w_in, n)):
+        proj = torch.empty(T, n_mix, dtype=h.dtype, device=x.device)
+        router = torch.empty(T, n_router, dtype=torch.float32,
+                             device=x.device) if n_router else None
+        if h.inside:
+            _lib().fei_gemv_parallel_in(
+                _p(proj), _p(router), _p(x), _p(w_in), _p(norm.gain), norm.eps,
+                _p(act), act.stride(0), T, n_mix, n_router, n, K, _stream())
+        else:
+            _lib().fei_gemm_m8_parallel_in(
+                _p(proj), _p(router), _p(h.rows), _p(w_in), _p(act),
+                act.stride(0), T, n_mix, n_router, n, K, _stream())
+        return proj, router
+    rows = h.rows
+    proj = torch.nn.functional.linear(rows, w_in[:n_mix])
+    if ff:
+        up = torch.nn.functional.linear(rows, w_in[n_mix:])
+        if not x.is_cuda:
+            act.copy_(ref.square_relu(up))
+        elif T:
+            _lib().fei_relu2_rows(_p(act), act.stride(0), _p(up),
+                                  up.stride(0), T, ff, _f32(up), _stream())
+    router = _mm_f32(rows, w_in[n_mix:], None) if n_router else None
+    return proj, router
+
+
+def gain_logits(h: GainNormed, w: torch.Tensor) -> torch.Tensor:
+    """normed rows @ w^T, float32."""
+    if not h.inside:
+        return logits_head(h.rows, w, 1.0, None)
+    T, K = h.x.shape
+    out = torch.empty(T, w.shape[0], dtype=torch.float32, device=w.device)
+    _lib().fei_gemv_gain(_p(out), _p(h.x.contiguous()), _p(w),
+                         _p(h.norm.gain), h.norm.eps, T, w.shape[0], K,
+                         _stream())
+    return out
+
+
 def _mm_f32(a: torch.Tensor, w: torch.Tensor,
             add: Optional[torch.Tensor]) -> torch.Tensor:
     """a @ w^T (+ add) with a float32 result; a 2-d ``add`` may be
@@ -159,19 +267,22 @@ def _mm_f32(a: torch.Tensor, w: torch.Tensor,
     return torch.addmm(add, a, w.t(), out_dtype=torch.float32, out=add)
 
 
-def residual_linear(x: torch.Tensor, a: torch.Tensor,
-                    w: torch.Tensor) -> torch.Tensor:
-    """x + a @ w^T, float32; x may be overwritten with it."""
+def residual_linear(x: torch.Tensor, a: torch.Tensor, w: torch.Tensor,
+                    mult: float = 1.0) -> torch.Tensor:
+    """x + mult * (a @ w^T), float32; x may be overwritten with it."""
     T, K = a.shape
     if a.is_cuda and _m8(T, K, a, w.shape[0]):
         _lib().fei_gemm_m8_f32(_p(x), _p(a), _p(w), None, T, w.shape[0], K, 1,
-                               1.0, 0.0, _stream())
+                               mult, 0.0, _stream())
         return x
     if a.is_cuda and _gemv_rows(T, K, a):
         _lib().fei_gemv_f32(_p(x), _p(a), _p(w), None, T, w.shape[0], K, 1,
-                            1.0, 0.0, 1, _stream())
+                            mult, 0.0, 1, _stream())
         return x
-    return _mm_f32(a, w, x)
+    if not a.is_cuda or a.dtype == torch.float32:
+        return x + mult * _mm_f32(a, w, None)
+    return torch.addmm(x, a, w.t(), out_dtype=torch.float32, alpha=mult,
+                       out=x)
 
 
 def linear_f32(a: torch.Tensor, w: torch.Tensor,

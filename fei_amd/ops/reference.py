@@ -377,3 +377,57 @@ def gla_gate_out(o, g, norm_w, eps):
     y = (rms(o, eps) * norm_w).flatten(1)
     gf = g.float()
     return y * (gf * torch.sigmoid(gf))
+
+
+def short_conv(u, first, weights):
+    """u [n, channels] float32, the ``taps - 1`` projections before it in
+    ``first`` (zeros before the sequence's start), weights [taps, channels]."""
+    taps = weights.shape[0]
+    ext = torch.cat([first, u])
+    y = torch.zeros_like(u)
+    for j in range(taps):
+        y = y + weights[j] * ext[j:j + u.shape[0]]
+    return y
+
+
+def sigmoid_attend(q, pos, keys, k0, m, bias):
+    """q [n, H, dim] at positions ``pos`` [n]; keys [N, row_width] cached rows
+    of positions k0 .. k0+N-1; bias [3, H]: r1, r2, pb. Returns [n, H, vdim]."""
+    N, G = keys.shape[0], m.kv_heads
+    k = keys[:, :G * m.dim].float().view(N, G, m.dim)
+    v = keys[:, G * m.dim:].float().view(N, G, m.vdim)
+    k, v = (t.repeat_interleave(m.heads // G, dim=1) for t in (k, v))
+    s = torch.einsum("nhd,khd->hnk", q, k) * m.scale
+    d = pos.long().view(-1, 1) - torch.arange(k0, k0 + N).view(1, -1)
+    r1, r2, pb = (b.view(-1, 1, 1) for b in bias)
+    s = s - r1 * torch.log(1.0 + r2 * d.clamp(min=0).float()) + pb
+    hide = d < 0
+    if m.window is not None:
+        hide = hide | (d >= m.window)
+    w = torch.sigmoid(s).masked_fill(hide, 0.0)
+    return torch.einsum("hnk,khd->nhd", w, v)
+
+
+def square_relu(x):
+    return torch.relu(x.float()).square()
+
+
+def route(logits, top, scale):
+    """Sigmoid router: (experts [T, top], weights [T, top] float32)."""
+    s = torch.sigmoid(logits.float())
+    ids = torch.topk(logits.float(), top, dim=-1).indices
+    w = s.gather(1, ids)
+    return ids, w / (w.sum(-1, keepdim=True) + 1e-20) * scale
+
+
+def moe(h, ids, weights, up, down):
+    """sum_k weights[t, k] * down[e] relu(up[e] h[t])^2, e = ids[t, k];
+    float32."""
+    out = torch.zeros(h.shape[0], down.shape[1])
+    for e in range(up.shape[0]):
+        t, k = (ids == e).nonzero(as_tuple=True)
+        if t.numel():
+            a = square_relu(torch.nn.functional.linear(h[t], up[e]))
+            y = torch.nn.functional.linear(a.to(h.dtype), down[e]).float()
+            out.index_add_(0, t, y * weights[t, k].unsqueeze(1))
+    return out
