@@ -16,8 +16,8 @@ from concurrent.futures import ThreadPoolExecutor
 CSRC = os.path.join(os.path.dirname(os.path.abspath(__file__)), "csrc")
 OUT = os.path.join(os.path.dirname(os.path.abspath(__file__)), "libfei_kernels.so")
 SOURCES = ["fei_kernels.hip", "attn_prefill.hip", "gemv.hip", "attn_decode_fused.hip", "gemv_fp8.hip", "stream_layer.hip",
-           "hybrid.hip", "latent_attn.hip", "gla.hip"]
-HEADERS = ["fei_common.h", "fei_epilogue.h", "fei_mma.h"]
+           "hybrid.hip", "latent_attn.hip", "gla.hip", "sigmoid_attn.hip", "moe.hip"]
+HEADERS = ["fei_common.h", "fei_epilogue.h", "fei_mma.h", "fei_attn.h"]
 HIPCC = os.environ.get("HIPCC", "hipcc")
 ARCH = os.environ.get("FEI_AMD_ARCH", "gfx950")
 # Packed fp32 VALU instructions are off: some of their forms have returned

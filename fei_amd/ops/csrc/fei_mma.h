@@ -36,6 +36,10 @@ template <> struct El<u16> {
   static __device__ __forceinline__ float exb(float x) {
     return __builtin_amdgcn_exp2f(x);
   }
+  static __device__ __forceinline__ float ln(float x) { return __logf(x); }
+  static __device__ __forceinline__ float inv(float x) {
+    return __builtin_amdgcn_rcpf(x);
+  }
 };
 template <> struct El<float> {
   typedef f32x8 frag;
@@ -44,6 +48,8 @@ template <> struct El<float> {
   static __device__ __forceinline__ float ex(float x) { return expf(x); }
   static constexpr float base = 1.f;
   static __device__ __forceinline__ float exb(float x) { return expf(x); }
+  static __device__ __forceinline__ float ln(float x) { return logf(x); }
+  static __device__ __forceinline__ float inv(float x) { return 1.f / x; }
 };
 
 // 8 consecutive elements at p (16-byte aligned in LDS and, where used, in

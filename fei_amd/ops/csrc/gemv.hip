@@ -513,7 +513,7 @@ k_gemm_m8(void* __restrict__ outp, const u16* __restrict__ x,
       float v = cred[0][m][n] + cred[1][m][n] + cred[2][m][n] + cred[3][m][n];
 #pragma unroll
       for (int c = 4; c < NW; ++c) v += cred[c][m][n];
-      epilogue<EPI>(outp, (long)m * N + n0 + n, n0 + n, v, ep);
+      epilogue<EPI>(outp, m, N, n0 + n, v, ep);
     }
   }
 }
@@ -541,6 +541,24 @@ extern "C" void fei_gemm_m8_f32(void* out, const void* x, const void* w,
   if (residual) BY_NW(EPI_RES); else BY_NW(EPI_F32);
 #undef BY_NW
 #undef M8
+}
+
+// All products of a parallel layer's input (see EPI_PARALLEL).
+extern "C" void fei_gemm_m8_parallel_in(void* out, float* router,
+                                        const void* x, const void* w,
+                                        void* act, long as, int M, int n_mix,
+                                        int n_router, int N, int K,
+                                        hipStream_t stream) {
+  const Epilogue ep{nullptr, 1.f,    0.f,       n_mix,
+                    n_router, router, (u16*)act, as};
+  if (N <= 8192)
+    hipLaunchKernelGGL((k_gemm_m8<false, EPI_PARALLEL, 8>),
+                       dim3(N / GEMM_NT), dim3(512), 0, stream, out,
+                       (const u16*)x, (const u16*)w, M, N, K, ep);
+  else
+    hipLaunchKernelGGL((k_gemm_m8<false, EPI_PARALLEL, 4>),
+                       dim3(N / GEMM_NT), dim3(256), 0, stream, out,
+                       (const u16*)x, (const u16*)w, M, N, K, ep);
 }
 
 extern "C" void fei_gemm_m8(void* out, const void* x, const void* w, int M,

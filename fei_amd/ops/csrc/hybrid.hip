@@ -1,5 +1,5 @@
 // Row-wise kernels and skinny products of decoders made of unlike layers
-// (models/tobarax.py): a float32 residual, two norms of the same rows, one
+// (models/tobarax.py, models/bokenex.py): a float32 residual, two norms of the same rows, one
 // stacked product for everything a layer reads, one product over the
 // concatenated mixer and feed-forward outputs that adds to the residual.
 // T is the element type of rows: u16 (bfloat16 bits) or float.
@@ -207,14 +207,111 @@ k_gemv_f32(float* __restrict__ out, const u16* __restrict__ x,
     if (threadIdx.x >= 2 * M) return;
     const int m = threadIdx.x >> 1, n = threadIdx.x & 1;
     if (n == 1 && n1 == n0) return;
-    epilogue<EPI>(out, (long)m * N + n0 + n, n0 + n,
+    epilogue<EPI>(out, m, N, n0 + n,
                   (red[0][n][m] + red[1][n][m]) + (red[2][n][m] + red[3][n][m]),
                   ep);
   } else if (lane == 0) {
 #pragma unroll
     for (int m = 0; m < M; ++m) {
-      epilogue<EPI>(out, (long)m * N + n0, n0, a0[m], ep);
-      if (n1 > n0) epilogue<EPI>(out, (long)m * N + n1, n1, a1[m], ep);
+      epilogue<EPI>(out, m, N, n0, a0[m], ep);
+      if (n1 > n0) epilogue<EPI>(out, m, N, n1, a1[m], ep);
+    }
+  }
+}
+
+// The same of rows under an RMS norm with one gain: x float32 as it is, the
+// sums times gain / rms(x).
+template <int M, int EPI, int KSPLIT>
+__global__ void __launch_bounds__(256)
+k_gemv_gain(void* __restrict__ out, const float* __restrict__ x,
+            const u16* __restrict__ w, const float* __restrict__ gain,
+            float eps, int N, int K, Epilogue ep) {
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int n0 = (KSPLIT == 1 ? blockIdx.x * 4 + wid : blockIdx.x) * 2;
+  if (n0 >= N) return;
+  const int n1 = min(n0 + 1, N - 1);
+  const s16x8* w0 = (const s16x8*)(w + (long)n0 * K);
+  const s16x8* w1 = (const s16x8*)(w + (long)n1 * K);
+  float a[3][M];                           // two rows, sum of squares
+#pragma unroll
+  for (int m = 0; m < M; ++m) a[0][m] = a[1][m] = a[2][m] = 0.f;
+  for (int i = KSPLIT == 1 ? lane : threadIdx.x; i < (K >> 3);
+       i += KSPLIT * 64) {
+    const s16x8 v0 = __builtin_nontemporal_load(w0 + i);
+    const s16x8 v1 = __builtin_nontemporal_load(w1 + i);
+#pragma unroll
+    for (int m = 0; m < M; ++m) {
+      const f32x8 xv = ld8(x + (long)m * K + i * 8);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        a[0][m] = fmaf(xv[j], bf2f((u16)v0[j]), a[0][m]);
+        a[1][m] = fmaf(xv[j], bf2f((u16)v1[j]), a[1][m]);
+        a[2][m] = fmaf(xv[j], xv[j], a[2][m]);
+      }
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < 3; ++i)
+#pragma unroll
+    for (int m = 0; m < M; ++m) a[i][m] = wave_reduce_sum(a[i][m]);
+  if (KSPLIT > 1) {
+    __shared__ float red[4][3][M];
+    if (lane == 0) {
+#pragma unroll
+      for (int i = 0; i < 3; ++i)
+#pragma unroll
+        for (int m = 0; m < M; ++m) red[wid][i][m] = a[i][m];
+    }
+    __syncthreads();
+    if (threadIdx.x >= 2 * M) return;
+    const int m = threadIdx.x >> 1, n = threadIdx.x & 1;
+    if (n == 1 && n1 == n0) return;
+    const float ss = (red[0][2][m] + red[1][2][m]) +
+                     (red[2][2][m] + red[3][2][m]);
+    epilogue<EPI>(out, m, N, n0 + n,
+                  ((red[0][n][m] + red[1][n][m]) +
+                   (red[2][n][m] + red[3][n][m])) *
+                      (*gain / sqrtf(ss / (float)K + eps)), ep);
+  } else if (lane == 0) {
+#pragma unroll
+    for (int m = 0; m < M; ++m) {
+      const float inv = *gain / sqrtf(a[2][m] / (float)K + eps);
+      epilogue<EPI>(out, m, N, n0, a[0][m] * inv, ep);
+      if (n1 > n0) epilogue<EPI>(out, m, N, n1, a[1][m] * inv, ep);
+    }
+  }
+}
+
+// out[t] = emb[tok[t]] + pos_emb[pos[t]]
+template <typename T, typename I>
+__global__ void __launch_bounds__(256)
+k_embed_pos(float* __restrict__ out, const I* __restrict__ tok,
+            const int* __restrict__ pos, const T* __restrict__ emb,
+            const T* __restrict__ pos_emb, int C) {
+  const int t = blockIdx.x, c = blockIdx.y * 256 + threadIdx.x;
+  if (c < C)
+    out[(long)t * C + c] = El<T>::ld(emb[(long)tok[t] * C + c]) +
+                           El<T>::ld(pos_emb[(long)pos[t] * C + c]);
+}
+
+// act = relu(up)^2
+template <typename T>
+__global__ void __launch_bounds__(256)
+k_relu2_rows(T* __restrict__ act, long as, const T* __restrict__ up, long us,
+             int rows, int ff, int vec) {
+  const int nv = vec ? ff >> 3 : ff;
+  for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+       i < (long)rows * nv; i += (long)gridDim.x * blockDim.x) {
+    const long row = i / nv;
+    const int c = (int)(i - row * nv);
+    if (vec) {
+      const auto u = ld8(up + row * us + c * 8);
+      typename El<T>::frag o;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) o[j] = El<T>::st(relu2(get8(u, j)));
+      st8(act + row * as + c * 8, o);
+    } else {
+      act[row * as + c] = El<T>::st(relu2(El<T>::ld(up[row * us + c])));
     }
   }
 }
@@ -264,6 +361,36 @@ void fei_swiglu_rows(void* act, long as, const void* gu, long gs, int rows,
                        (u16*)act, as, (const u16*)gu, gs, rows, ff, vec);
 }
 
+// bits: 1 = float32 rows, 2 = 64-bit token ids
+void fei_embed_pos(float* out, const void* tok, const int* pos,
+                   const void* emb, const void* pos_emb, int T, int C,
+                   int bits, hipStream_t stream) {
+  const dim3 grid(T, (C + 255) / 256);
+#define EMB(E, I)                                                           \
+  hipLaunchKernelGGL((k_embed_pos<E, I>), grid, dim3(256), 0, stream, out,  \
+                     (const I*)tok, pos, (const E*)emb, (const E*)pos_emb, C)
+  switch (bits) {
+    case 0: EMB(u16, int); break;
+    case 1: EMB(float, int); break;
+    case 2: EMB(u16, long); break;
+    default: EMB(float, long); break;
+  }
+#undef EMB
+}
+
+void fei_relu2_rows(void* act, long as, const void* up, long us, int rows,
+                    int ff, int f32, hipStream_t stream) {
+  const int vec = ff % 8 == 0 && as % 8 == 0 && us % 8 == 0 &&
+                  (size_t)act % 16 == 0 && (size_t)up % 16 == 0;
+  const dim3 grid(grid_for((long)rows * ff, vec ? 2048 : 256));
+  if (f32)
+    hipLaunchKernelGGL(k_relu2_rows<float>, grid, dim3(256), 0, stream,
+                       (float*)act, as, (const float*)up, us, rows, ff, vec);
+  else
+    hipLaunchKernelGGL(k_relu2_rows<u16>, grid, dim3(256), 0, stream,
+                       (u16*)act, as, (const u16*)up, us, rows, ff, vec);
+}
+
 void fei_softcap(float* y, long n, float scale, float cap,
                  hipStream_t stream) {
   hipLaunchKernelGGL(k_softcap, dim3(grid_for(n, 1024)), dim3(256), 0, stream,
@@ -297,7 +424,43 @@ void fei_gemv_mix_in(void* proj, void* act, const void* x1, const void* x2,
 #undef CALL
 }
 
-// residual != 0: out += x w^T; else out = softcap(x w^T * scale, cap) + bias.
+// Products of one or two rows under a norm with one gain, K % 8 == 0.
+#define GAIN(EPI)                                                           \
+  do {                                                                      \
+    if (M == 1) {                                                           \
+      if (share) GAIN_(1, EPI, 4); else GAIN_(1, EPI, 1);                   \
+    } else if (M == 2) {                                                    \
+      if (share) GAIN_(2, EPI, 4); else GAIN_(2, EPI, 1);                   \
+    }                                                                       \
+  } while (0)
+#define GAIN_(MV, EPI, KSP)                                                 \
+  hipLaunchKernelGGL((k_gemv_gain<MV, EPI, KSP>), grid, dim3(256), 0,       \
+                     stream, out, x, (const u16*)w, gain, eps, N, K, ep)
+
+void fei_gemv_gain(void* out, const float* x, const void* w,
+                   const float* gain, float eps, int M, int N, int K,
+                   hipStream_t stream) {
+  const bool share = N < 8192;
+  const dim3 grid(share ? (N + 1) / 2 : (N + 7) / 8);
+  const Epilogue ep{nullptr, 1.f, 0.f};
+  GAIN(EPI_F32);
+}
+
+// All products of a parallel layer's input (see EPI_PARALLEL).
+void fei_gemv_parallel_in(void* out, float* router, const float* x,
+                          const void* w, const float* gain, float eps,
+                          void* act, long as, int M, int n_mix, int n_router,
+                          int N, int K, hipStream_t stream) {
+  const bool share = N < 8192;
+  const dim3 grid(share ? (N + 1) / 2 : (N + 7) / 8);
+  const Epilogue ep{nullptr, 1.f,    0.f,       n_mix,
+                    n_router, router, (u16*)act, as};
+  GAIN(EPI_PARALLEL);
+}
+#undef GAIN
+#undef GAIN_
+
+// residual != 0: out += scale x w^T; else out = softcap(x w^T * scale, cap) + bias.
 void fei_gemv_f32(void* out, const void* x, const void* w, const float* bias,
                   int M, int N, int K, int residual, float scale, float cap,
                   int nt, hipStream_t stream) {

@@ -12,6 +12,7 @@
 // T is u16 (bfloat16 bits) or float. Scores, weights and sums are float32;
 // where a weight enters a bfloat16 matrix product it is given as a high and a
 // low part, so that it keeps about 16 bits.
+#include "fei_attn.h"
 #include "fei_common.h"
 #include "fei_mma.h"
 
@@ -24,17 +25,6 @@ struct Geo {           // sizes of one mixer
   float scale;
   int window;          // keys a query sees, itself included; 0 = all
 };
-
-__device__ __forceinline__ int first_key(int pos, int window) {
-  return window > 0 && pos >= window ? pos - window + 1 : 0;
-}
-
-__device__ __forceinline__ long cache_row(const int* __restrict__ table,
-                                          int W, int seq, int pos,
-                                          int bs_log) {
-  return ((long)table[(long)seq * W + (pos >> bs_log)] << bs_log) +
-         (pos & ((1 << bs_log) - 1));
-}
 
 // Norm of the latent and rotation of the shared key part of one token, into
 // its cache row. ``ckr`` points at the row's kr + rot projected values.
@@ -163,16 +153,6 @@ k_latent_absorb(const T* __restrict__ proj, long ps, T* __restrict__ qa,
     for (int i = 0; i < 16; ++i) v += part[i][tid];
     qo[c] = El<T>::st(v);
   }
-}
-
-// P as operand: one part for float, a high and a low one for bfloat16.
-template <typename T> struct Parts { static constexpr int n = 1; };
-template <> struct Parts<u16> { static constexpr int n = 2; };
-
-template <typename T>
-__device__ __forceinline__ T part_of(float v, int i) {
-  const T hi = El<T>::st(v);
-  return i == 0 ? hi : El<T>::st(v - El<T>::ld(hi));
 }
 
 // Decode partials. grid (splits, ceil(heads / 16 NH), B). The visible
@@ -481,14 +461,6 @@ k_latent_gather(T* __restrict__ c, T* __restrict__ kr_out,
     for (int j = threadIdx.x; j < g.rot; j += blockDim.x)
       kr_out[(long)i * g.rot + j] = src[g.kr + j];
   }
-}
-
-// Place of (column, key) in the transposed value tile: 64 keys a column in
-// blocks of 8, the block index permuted by the column so that neither the
-// stores (lanes along columns) nor the reads (16 columns, one block) pile up
-// on a bank.
-__device__ __forceinline__ int vt_at(int col, int key) {
-  return col * 64 + ((((key >> 3) ^ col ^ (col >> 3)) & 7) << 3) + (key & 7);
 }
 
 // Flash attention of prompt portions over expanded keys and values.

@@ -25,8 +25,8 @@ MAX_EXPERTS = 1024
 
 def declare(lib: ctypes.CDLL) -> None:
     lib.fei_moe_route.argtypes = [_vp] * 3 + [_i] * 3 + [_f, _vp]
-    lib.fei_moe_plan.argtypes = [_vp] * 6 + [_i] * 5 + [_vp]
-    lib.fei_moe_gemm.argtypes = [_vp] * 6 + [_i] * 7 + [_vp]
+    lib.fei_moe_plan.argtypes = [_vp] * 5 + [_i] * 5 + [_vp]
+    lib.fei_moe_gemm.argtypes = [_vp] * 6 + [_i] * 5 + [_vp]
     lib.fei_moe_add.argtypes = [_vp] * 4 + [_i] * 3 + [_f, _i, _vp]
     lib.fei_moe_up_gemv.argtypes = (
         [_vp] * 6 + [_i] + [_vp, _f] + [_i] * 5 + [_f, _vp])
@@ -98,14 +98,14 @@ def residual_moe(x: torch.Tensor, h: GainNormed, router: torch.Tensor,
     tiles, count = meta[2 * n:-1], meta[-1:]
     # order: row of every slot, slots sorted by expert; place: slot of (t, k)
     lib.fei_moe_plan(_p(order), _p(place), _p(tiles), _p(count), _p(ids),
-                     None, n, E, f.top, rows, max_tiles, st)
+                     n, E, f.top, rows, max_tiles, st)
     act = torch.empty(n, ff, dtype=up.dtype, device=dev)
     y = torch.empty(n, C, dtype=up.dtype, device=dev)
     bits = _f32(up) | (2 if big else 0)
     lib.fei_moe_gemm(_p(act), _p(h.rows), _p(up), _p(order), _p(tiles),
-                     _p(count), max_tiles, ff, C, E, n, 1, bits, st)
+                     _p(count), max_tiles, ff, C, 1, bits, st)
     lib.fei_moe_gemm(_p(y), _p(act), _p(down), None, _p(tiles), _p(count),
-                     max_tiles, C, ff, E, n, 0, bits, st)
+                     max_tiles, C, ff, 0, bits, st)
     x = residual_linear(x, a, w_o, mult)
     lib.fei_moe_add(_p(x), _p(y), _p(place), _p(w), T, C, f.top, mult,
                     _f32(up), st)

@@ -30,7 +30,7 @@ def declare(lib: ctypes.CDLL) -> None:
     lib.fei_sig_conv.argtypes = (
         [_vp, _vp, _l] + [_vp] * 10 + [_i] * 10 + [_f, _i, _vp])
     lib.fei_sig_prefill.argtypes = (
-        [_vp, _l] + [_vp] * 6 + [_i] * 9 + [_f, _i, _i, _vp])
+        [_vp, _l] + [_vp] * 6 + [_i] * 9 + [_f, _i, _vp])
 
 
 def check_sigmoid_geometry(m) -> None:
@@ -124,4 +124,4 @@ def sigmoid_attn_prefill(proj, out, m, w, batch, rows, states,
     _lib().fei_sig_prefill(
         _p(out), out.stride(0), _p(q), _p(rows), _p(w.bias), _p(spans),
         _p(tiles), _p(batch.table), tiles.shape[0], n, W, bs_log, m.heads,
-        m.kv_heads, m.dim, m.vdim, m.window or 0, m.scale, _f32(proj), 0, st)
+        m.kv_heads, m.dim, m.vdim, m.window or 0, m.scale, _f32(proj), st)
