@@ -40,8 +40,9 @@ def short_conv(u, w):
     return y
 
 
-def distance_bias(i, j, r1, r2):
-    return r1 * math.log(1.0 + r2 * (i - j))
+def distance_bias(d, r1, r2):
+    """Taken off the score of a key d positions back."""
+    return r1 * torch.log(1.0 + r2 * d)
 
 
 def visible_keys(i, window):
@@ -51,8 +52,8 @@ def visible_keys(i, window):
 
 def key_weights(i, q, k, keys, scale, r1, r2, pb):
     """Weights of ``keys`` for the query q of position i; k [T, dim]."""
-    bias = torch.tensor([distance_bias(i, j, r1, r2) for j in keys],
-                        dtype=real)
+    d = i - torch.arange(keys.start, keys.stop, dtype=real)
+    bias = distance_bias(d, r1, r2)
     return torch.sigmoid(k[keys.start:keys.stop] @ q * scale - bias + pb)
 
 
@@ -135,3 +136,72 @@ def greedy(tokens, n, W, cfg):
     for _ in range(n):
         ids.append(int(forward(ids, W, cfg)[-1].argmax()))
     return ids[len(tokens):]
+
+
+# -- random models -----------------------------------------------------------
+
+def tensor_shapes(cfg):
+    """name -> shape of every tensor of a model with this configuration."""
+    C = cfg["width"]
+    out = {"embed": (cfg["vocab"], C), "pos": (cfg["max_positions"], C),
+           "final.norm": (), "head": (cfg["vocab"], C)}
+    for i, L in enumerate(cfg["layers"]):
+        p, m, f = f"l{i}.", L["mixer"], L.get("mlp")
+        H, G = m["heads"], m["kv_heads"]
+        out[p + "norm1"] = ()
+        for n, rows in (("q", H * m["dim"]), ("k", G * m["dim"]),
+                        ("v", G * m["vdim"])):
+            out[p + "mix." + n] = (rows, C)
+            out[p + "mix." + n + ".conv"] = (rows, m["conv"])
+        for n, size in (("q.norm", m["dim"]), ("k.norm", m["dim"]),
+                        ("r1", H), ("r2", H), ("pb", H)):
+            out[p + "mix." + n] = (size,)
+        out[p + "mix.o"] = (C, H * m["vdim"])
+        if not f:
+            continue
+        if f["kind"] == "dense":
+            names, ff = [p + "mlp."], f["ff"]
+        else:
+            E, ff = f["router"]["experts"], f["expert"]["ff"]
+            names = [f"{p}mlp.e{e}." for e in range(E)]
+            out[p + "mlp.router"] = (E, C)
+        for n in names:
+            out[n + "up"] = (ff, C)
+            out[n + "down"] = (C, ff)
+    return out
+
+
+def random_weights(cfg, seed):
+    """bfloat16-valued float64 weights: gains around 1, distance biases of
+    unlike strength, key weights around a tenth."""
+    g = torch.Generator().manual_seed(seed)
+    W = {}
+    for name, shape in tensor_shapes(cfg).items():
+        t = torch.randn(shape, generator=g)
+        if name.endswith(("norm", "norm1")):
+            t = 1.0 + 0.3 * t
+        elif name.endswith(".r1"):
+            t = t.abs()
+        elif name.endswith(".r2"):
+            t = 0.05 + 0.3 * t.abs()
+        elif name.endswith(".pb"):
+            t = -2.0 + 0.5 * t
+        elif name.endswith(".conv"):
+            t = t / math.sqrt(shape[-1])
+        elif name.endswith("router"):
+            t = t * (3.0 / math.sqrt(shape[-1]))   # choices far from a tie
+        elif name in ("embed", "pos"):
+            t = 0.7 * t
+        else:
+            t = t * (1.3 / math.sqrt(shape[-1]))
+        W[name] = t.bfloat16().to(real)
+    return W
+
+
+def save_model(path, cfg, W):
+    from safetensors.torch import save_file
+    os.makedirs(path, exist_ok=True)
+    save_file({k: v.bfloat16().contiguous() for k, v in W.items()},
+              os.path.join(path, "model.safetensors"))
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(cfg, f)

@@ -14,16 +14,15 @@ import numpy as np
 import pytest
 import torch
 
+import step_helpers
 import tobarax_oracle as oracle
 from fei_amd import ops
 from fei_amd.engine.config import MODEL_SPECS, TobaraxSpec, get_spec
 from fei_amd.engine.kv_cache import HybridCache
-from fei_amd.engine.step import StepEntry, StepRunner
-from fei_amd.models import model_class
+from fei_amd.engine.step import StepEntry
 from fei_amd.models.tobarax import TobaraxModel
-
-DEVICES = ["cpu", pytest.param("cuda", marks=pytest.mark.gpu)]
-F32_TOL = 3e-5
+from step_helpers import (DEVICES, F32_TOL, err, run, run_mixed,
+                          serve_sessions, toks)
 
 
 def att(heads=3, dim=20, rot=6, vdim=28, kr=44, window=37, scale=None,
@@ -69,58 +68,10 @@ CONFIGS = {
 }
 
 
-class Net:
-    """A model with its oracle weights."""
-
-    def __init__(self, tmp, cfg, seed=0, device="cpu", dtype=torch.float32,
-                 edit=None, max_seq=512, gate_rank=5):
-        self.cfg = cfg
-        self.W = oracle.random_weights(cfg, seed, gate_rank)
-        if edit:
-            edit(self.W)
-            self.W = {k: v.bfloat16().to(oracle.real)
-                      for k, v in self.W.items()}
-        self.path = str(tmp)
-        oracle.save_model(self.path, cfg, self.W)
-        spec = get_spec(self.path)
-        self.model = model_class(spec)(spec, torch.device(device), dtype,
-                                       max_seq_len=max_seq,
-                                       weights=self.path)
-
-    def runner(self, blocks=16, slots=4, block_size=64, poison=True):
-        r = StepRunner(self.model, blocks, slots, block_size)
-        if poison:        # whatever is read without having been written shows
-            for t in r.cache.rows + r.cache.states:
-                if t is not None:
-                    t.fill_(float("nan"))
-        return r
-
-    def want(self, tokens):
-        return oracle.forward(tokens, self.W, self.cfg)
-
-
-def toks(n, vocab, seed):
-    g = torch.Generator().manual_seed(seed)
-    return torch.randint(0, vocab, (n,), generator=g).tolist()
-
-
-def err(got, want):
-    """Largest row error, relative to the rows' size."""
-    got, want = got.double().cpu(), want.double()
-    assert got.shape == want.shape
-    d = (got - want).pow(2).mean(-1).sqrt()
-    return float((d / want.pow(2).mean(-1).sqrt()).max())
-
-
-def run(r, sid, tokens, sizes):
-    """All logits of ``tokens`` run in portions of ``sizes`` (repeated)."""
-    out, at, i = [], 0, 0
-    while at < len(tokens):
-        part = tokens[at:at + sizes[i % len(sizes)]]
-        out.append(r.step([StepEntry(sid, part, range(len(part)))]))
-        at += len(part)
-        i += 1
-    return torch.cat(out)
+def Net(tmp, cfg, seed=0, device="cpu", dtype=torch.float32, edit=None,
+        max_seq=512, gate_rank=5):
+    return step_helpers.Net(tmp, oracle, cfg, seed, device, dtype, edit,
+                            max_seq, gate_rank=gate_rank)
 
 
 # -- mechanisms alone ------------------------------------------------------------
@@ -442,35 +393,9 @@ def test_mixed_batches(tmp_path, name, device):
     reqs = {i: toks(n, V, 30 + i) for i, n in enumerate((150, 97, 64, 33, 120))}
     want = {i: net.want(t) for i, t in reqs.items()}
     r = net.runner(blocks=8, slots=3)
-    rng = np.random.default_rng(0)
-    at = {i: 0 for i in reqs}
-    live, waiting = {}, list(reqs)
-    got = {i: [] for i in reqs}
-    while live or waiting:
-        while waiting and r.cache.free_slots() and \
-                len(reqs[waiting[0]]) + 64 <= r.cache.free_blocks() * 64:
-            live[waiting[0]] = r.admit(len(reqs[waiting[0]]))
-            waiting.pop(0)
-        entries, who = [], []
-        for i, sid in live.items():
-            if len(live) > 1 and rng.random() < 0.2:
-                continue
-            n = int(rng.choice([1, 1, 2, 3, 17, 64, 70]))
-            part = reqs[i][at[i]:at[i] + n]
-            entries.append(StepEntry(sid, part, range(len(part))))
-            who.append((i, len(part)))
-        if not entries:
-            continue
-        logits = r.step(entries)
-        row = 0
-        for i, n in who:
-            got[i].append(logits[row:row + n])
-            row += n
-            at[i] += n
-            if at[i] == len(reqs[i]):
-                r.release(live.pop(i))
+    got = run_mixed(r, reqs)
     for i in reqs:
-        assert err(torch.cat(got[i]), want[i]) < F32_TOL, i
+        assert err(got[i], want[i]) < F32_TOL, i
     assert r.cache.free_blocks() == 8 and r.cache.free_slots() == 3
 
 
@@ -698,22 +623,7 @@ def test_sessions(tmp_path, device):
     mgr.eos = -1                       # run to the length asked for
     prompts = [toks(n, 272, 40 + n) for n in (50, 3, 90, 20, 61)]
     want = [oracle.greedy(p, 15, net.W, GEN) for p in prompts]
-    todo, open_, got = list(range(5)), {}, {}
-    for _ in range(200):
-        while todo:
-            try:
-                open_[todo[0]] = mgr.open(prompts[todo[0]], max_new_tokens=15)
-                todo.pop(0)
-            except MemoryError:
-                break
-        if mgr.step_chunk(3) == 0:
-            break
-        for i, sid in list(open_.items()):
-            if mgr.result(sid)["done"]:
-                got[i] = mgr.result(sid)["token_ids"]
-                mgr.close(sid)
-                del open_[i]
-    assert [got.get(i) for i in range(5)] == want
+    assert serve_sessions(mgr, prompts, 15) == want
     assert mgr.pool.free_blocks() == 6 and mgr.pool.free_slots() == 3
 
 
