@@ -2,8 +2,8 @@
 
 ``BlockAllocator`` hands out fixed-size blocks; what lies in a block is the
 subclass's: ``PagedKVPool`` keys and values of one attention layer per entry,
-``HybridCache`` one row per token for every latent-attention layer run and,
-beside the blocks, a slot of recurrent state for every linear-attention one.
+``HybridCache`` one row per token for every layer run that caches rows and,
+beside the blocks, a slot of state for every one that keeps some.
 
 Sized for MI355X's 288 GB HBM3E: the pool reserves a fraction of free GPU
 memory as fixed-size blocks; sequences map logical block indices to physical
@@ -144,11 +144,12 @@ class PagedKVPool(BlockAllocator):
 class HybridCache(BlockAllocator):
     """Cache of a decoder whose layer runs differ.
 
-    ``rows[r]`` (latent attention): [(num_blocks + 1) * block_size, width],
-    one row per token. ``states[r]`` (linear attention): float32
-    [num_slots + 1, *shape], one entry per live sequence. The other of the
-    two is None. A sequence holds one state slot from ``new_sequence`` to
-    ``release`` and as many blocks as its length needs.
+    ``rows[r]``: [(num_blocks + 1) * block_size, width], one row per token
+    (a latent; keys and values). ``states[r]``: float32
+    [num_slots + 1, *shape], one entry per live sequence (the state of linear
+    attention; the last inputs of a short convolution). Either is None where
+    the run's mixer has none. A sequence holds one state slot from
+    ``new_sequence`` to ``release`` and as many blocks as its length needs.
 
     The last block and the last slot belong to no sequence: they take the
     writes of steps that must leave no trace (graph warm-up).

@@ -40,9 +40,114 @@ __device__ __forceinline__ int channels(const Geo& g) {
   return g.heads * g.dim + g.kvh * (g.dim + g.vdim);
 }
 
+// Per-head norm of a group's LG x 8 values of which n count.
+template <int LG>
+__device__ __forceinline__ void head_norm(float (&y)[8], int n, float eps,
+                                          const float (&wn)[8]) {
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) ss = fmaf(y[j], y[j], ss);
+  ss = row16_sum(ss);
+  if (LG == 32) ss += __shfl_xor(ss, 16);
+  const float inv = 1.f / sqrtf(ss / (float)n + eps);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) y[j] *= inv * wn[j];
+}
+
 // Convolution and norms of prompt rows: queries to q, keys and values to
-// their cache rows. A group of LG lanes takes one head of one token, a lane
-// 8 of its channels. spans [.][3]: first row, rows, first position.
+// their cache rows. A group of LG lanes takes one head of RUN rows one after
+// another, a lane 8 of its channels: the weights and the TAPS - 1 projections
+// before a row stay in registers. spans [.][3]: first row, rows, first
+// position. Sizes are multiples of 8.
+constexpr int RUN = 8;
+
+template <typename T, int LG, int TAPS>
+__global__ void __launch_bounds__(256)
+k_sig_conv_run(T* __restrict__ q, const T* __restrict__ proj, long ps,
+               T* __restrict__ rows, const float* __restrict__ states,
+               Conv cv, const int* __restrict__ spans,
+               const int* __restrict__ row_seq, const int* __restrict__ pos,
+               const int* __restrict__ slots, const int* __restrict__ table,
+               int n_rows, int seq0, int W, int bs_log, Geo g) {
+  const int units = g.heads + 2 * g.kvh;
+  const int item = blockIdx.x * (256 / LG) + threadIdx.x / LG;
+  const int t0 = item / units * RUN, u = item % units;
+  if (t0 >= n_rows) return;                // whole groups
+  const int CH = channels(g), R = g.kvh * (g.dim + g.vdim);
+  const bool is_q = u < g.heads, is_v = u >= g.heads + g.kvh;
+  const int n = is_v ? g.vdim : g.dim;
+  const int ch0 = is_v ? (g.heads + g.kvh) * g.dim +
+                             (u - g.heads - g.kvh) * g.vdim
+                       : u * g.dim;
+  const int c = (threadIdx.x & (LG - 1)) * 8;
+  const bool on = c < n;
+  const int ch = ch0 + (on ? c : 0);
+  float w[TAPS][8], wn[8], past[TAPS][8];  // past[a]: a rows back; [0] unused
+#pragma unroll
+  for (int i = 0; i < TAPS; ++i) {
+    const f32x8 v = ld8(cv.w + (long)i * CH + ch);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) w[i][j] = v[j];
+  }
+  if (!is_v) {
+    const f32x8 v = ld8((is_q ? cv.qn : cv.kn) + (on ? c : 0));
+#pragma unroll
+    for (int j = 0; j < 8; ++j) wn[j] = v[j];
+  }
+  int last = -1;
+#pragma unroll
+  for (int k = 0; k < RUN; ++k) {
+    const int t = t0 + k;
+    if (t >= n_rows) return;
+    const int row = seq0 + t, seq = row_seq[row], p = pos[row];
+    if (seq != last) {                     // the run or a portion starts
+      last = seq;
+      const int row0 = spans[(seq - seq0) * 3];
+#pragma unroll
+      for (int a = 1; a < TAPS; ++a) {
+        if (row - a >= row0) {
+          const auto v = ld8(proj + (long)(row - a) * ps + ch);
+#pragma unroll
+          for (int j = 0; j < 8; ++j) past[a][j] = get8(v, j);
+        } else if (p - a >= 0) {
+          const f32x8 v = ld8(states + ((long)slots[seq] * TAPS +
+                                        (p - a) % TAPS) * CH + ch);
+#pragma unroll
+          for (int j = 0; j < 8; ++j) past[a][j] = v[j];
+        } else {
+#pragma unroll
+          for (int j = 0; j < 8; ++j) past[a][j] = 0.f;
+        }
+      }
+    }
+    const auto v = ld8(proj + (long)row * ps + ch);
+    float y[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const float x = get8(v, j);
+      y[j] = 0.f;
+#pragma unroll
+      for (int a = TAPS - 1; a > 0; --a)
+        y[j] = fmaf(w[TAPS - 1 - a][j], past[a][j], y[j]);
+      y[j] = on ? fmaf(w[TAPS - 1][j], x, y[j]) : 0.f;
+#pragma unroll
+      for (int a = TAPS - 1; a > 1; --a) past[a][j] = past[a - 1][j];
+      if (TAPS > 1) past[TAPS > 1 ? 1 : 0][j] = x;
+    }
+    if (!is_v) head_norm<LG>(y, n, cv.eps, wn);
+    if (on) {
+      T* dst = is_q ? q + (long)t * g.heads * g.dim + ch
+                    : rows + cache_row(table, W, seq, p, bs_log) * R +
+                          (ch - g.heads * g.dim);
+      typename El<T>::frag o;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) o[j] = El<T>::st(y[j]);
+      st8(dst, o);
+    }
+  }
+}
+
+// The same for any sizes and any number of taps, one row per group.
 template <typename T, int LG, bool VEC>
 __global__ void __launch_bounds__(256)
 k_sig_conv(T* __restrict__ q, const T* __restrict__ proj, long ps,
@@ -94,16 +199,11 @@ k_sig_conv(T* __restrict__ q, const T* __restrict__ proj, long ps,
     }
   }
   if (!is_v) {
-    float ss = 0.f;
+    const float* src = u < g.heads ? cv.qn : cv.kn;
+    float wn[8];
 #pragma unroll
-    for (int j = 0; j < 8; ++j) ss = fmaf(y[j], y[j], ss);
-    ss = row16_sum(ss);
-    if (LG == 32) ss += __shfl_xor(ss, 16);
-    const float inv = 1.f / sqrtf(ss / (float)n + cv.eps);
-    const float* wn = (u < g.heads ? cv.qn : cv.kn) + c;
-#pragma unroll
-    for (int j = 0; j < 8; ++j)
-      if (c + j < n) y[j] *= inv * wn[j];
+    for (int j = 0; j < 8; ++j) wn[j] = c + j < n ? src[c + j] : 0.f;
+    head_norm<LG>(y, n, cv.eps, wn);
   }
   if (c >= n) return;
   T* dst = u < g.heads
@@ -123,7 +223,8 @@ k_sig_conv(T* __restrict__ q, const T* __restrict__ proj, long ps,
   }
 }
 
-// State after the portions: their last projected rows. grid (portions, taps)
+// State after the portions: their last projected rows. grid (portions, taps,
+// ceil(channels / 256))
 template <typename T>
 __global__ void __launch_bounds__(256)
 k_sig_state(float* __restrict__ states, const T* __restrict__ proj, long ps,
@@ -134,9 +235,10 @@ k_sig_state(float* __restrict__ states, const T* __restrict__ proj, long ps,
   if (a >= n) return;
   const int p = sp[2] + n - 1 - a;
   const T* src = proj + (long)(sp[0] + n - 1 - a) * ps;
-  float* dst = states +
-               ((long)slots[seq0 + blockIdx.x] * taps + p % taps) * CH;
-  for (int i = threadIdx.x; i < CH; i += 256) dst[i] = El<T>::ld(src[i]);
+  const int i = blockIdx.z * 256 + threadIdx.x;
+  if (i < CH)
+    states[((long)slots[seq0 + blockIdx.x] * taps + p % taps) * CH + i] =
+        El<T>::ld(src[i]);
 }
 
 // Place of a key of a tile of 64 in the order of the second product.
@@ -460,6 +562,11 @@ k_sig_decode(T* __restrict__ out, long os, float* __restrict__ part,
   {
     float* st = states ? states + (long)slots[b] * cv.taps * CH : nullptr;
     const T* pr = proj + (long)b * ps;
+    const int newest = p % cv.taps;
+    auto ring = [&](int a) {               // place of the row a positions back
+      const int i = newest - a;
+      return i < 0 ? i + cv.taps : i;
+    };
     const int units = owner || split == 0 ? nh + 2 : nh;
     for (int u = w; u < units; u += 4) {
       const bool is_q = u < nh, is_v = u == nh + 1;
@@ -469,18 +576,35 @@ k_sig_decode(T* __restrict__ out, long os, float* __restrict__ part,
                                  (is_v ? g.kvh * g.dim + gk * g.vdim
                                        : gk * g.dim);
       const bool keep = st && split == 0 && (is_q || hy == 0);
-      float y[4], ss = 0.f;
+      // all loads of up to 4 taps before the first use
+      float x[4][4], cw[4][4], y[4], ss = 0.f;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int c = lane + 64 * i;
+        if (c < n) {
+          x[i][0] = El<T>::ld(pr[ch0 + c]);
+          cw[i][0] = cv.w[(long)(cv.taps - 1) * CH + ch0 + c];
+#pragma unroll
+          for (int a = 1; a < 4; ++a) {
+            x[i][a] = cw[i][a] = 0.f;
+            if (a < cv.taps && a <= p) {
+              x[i][a] = st[(long)ring(a) * CH + ch0 + c];
+              cw[i][a] = cv.w[(long)(cv.taps - 1 - a) * CH + ch0 + c];
+            }
+          }
+        }
+      }
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int c = lane + 64 * i;
         y[i] = 0.f;
         if (c < n) {
-          const float x = El<T>::ld(pr[ch0 + c]);
-          y[i] = x * cv.w[(long)(cv.taps - 1) * CH + ch0 + c];
-          for (int a = 1; a < cv.taps && a <= p; ++a)
+          for (int a = min(cv.taps - 1, p); a >= 4; --a)
             y[i] = fmaf(cv.w[(long)(cv.taps - 1 - a) * CH + ch0 + c],
-                        st[(long)((p - a) % cv.taps) * CH + ch0 + c], y[i]);
-          if (keep) st[(long)(p % cv.taps) * CH + ch0 + c] = x;
+                        st[(long)ring(a) * CH + ch0 + c], y[i]);
+#pragma unroll
+          for (int a = 3; a >= 0; --a) y[i] = fmaf(cw[i][a], x[i][a], y[i]);
+          if (keep) st[(long)ring(0) * CH + ch0 + c] = x[i][0];
           ss = fmaf(y[i], y[i], ss);
         }
       }
@@ -672,16 +796,34 @@ void run_conv(T* q, const T* proj, long ps, T* rows, float* states, Conv cv,
                      dim3((items + 256 / LG - 1) / (256 / LG)), dim3(256),   \
                      0, stream, q, proj, ps, rows, states, cv, spans,        \
                      row_seq, pos, slots, table, n_rows, seq0, W, bs_log, g)
-  if (small && vec) CONV(16, true);
+#define CONV_RUN(LG, TAPS)                                                   \
+  hipLaunchKernelGGL((k_sig_conv_run<T, LG, TAPS>),                          \
+                     dim3((runs + 256 / LG - 1) / (256 / LG)), dim3(256), 0, \
+                     stream, q, proj, ps, rows, states, cv, spans, row_seq,  \
+                     pos, slots, table, n_rows, seq0, W, bs_log, g)
+#define BY_LG(TAPS)                                              \
+  do {                                                           \
+    if (small) CONV_RUN(16, TAPS); else CONV_RUN(32, TAPS);      \
+  } while (0)
+  const long runs = (long)((n_rows + RUN - 1) / RUN) *
+                    (g.heads + 2 * g.kvh);
+  if (vec && cv.taps == 1) BY_LG(1);
+  else if (vec && cv.taps == 2) BY_LG(2);
+  else if (vec && cv.taps == 3) BY_LG(3);
+  else if (vec && cv.taps == 4) BY_LG(4);
+  else if (small && vec) CONV(16, true);
   else if (small) CONV(16, false);
   else if (vec) CONV(32, true);
   else CONV(32, false);
+#undef BY_LG
+#undef CONV_RUN
 #undef CONV
+  const int CH = g.heads * g.dim + g.kvh * (g.dim + g.vdim);
   if (states)
-    hipLaunchKernelGGL(k_sig_state<T>, dim3(n_portions, cv.taps), dim3(256),
+    hipLaunchKernelGGL(k_sig_state<T>,
+                       dim3(n_portions, cv.taps, (CH + 255) / 256), dim3(256),
                        0, stream, states, proj, ps, spans, slots, seq0,
-                       cv.taps,
-                       g.heads * g.dim + g.kvh * (g.dim + g.vdim));
+                       cv.taps, CH);
 }
 
 template <typename T, int KS, int DC>

@@ -486,6 +486,36 @@ def test_window_edge(tmp_path, window, conv, device):
                 assert err(logits(b, s)[q][None], new[None]) < F32_TOL, (q, s)
 
 
+@pytest.mark.gpu
+@pytest.mark.parametrize("window", [1, 31, 32, 33, 64, 100])
+def test_window_edge_in_bfloat16(tmp_path, window):
+    """The token before the first that a window reaches does not change a bit
+    of the logits; the first one does, as much as it should."""
+    conv = 2
+    cfg = make_cfg([(att(4, 1, 64, 64, window, conv), None)], width=32,
+                   vocab=71, mult=1.0)
+    net = Net(tmp_path, cfg, 20, "cuda", torch.bfloat16, edit=every_key_counts)
+    r = net.runner(slots=1)
+
+    def logits(tokens, sizes):
+        sid = r.admit()
+        out = run(r, sid, tokens, sizes)
+        r.release(sid)
+        return out
+    a = toks(200, cfg["vocab"], 19)
+    for q in (127, 128, 199):
+        k = q - window + 1 - (conv - 1)
+        b, c = list(a), list(a)
+        b[k] = (b[k] + 7) % cfg["vocab"]
+        c[k - 1] = (c[k - 1] + 7) % cfg["vocab"]
+        want = net.want(b)[q] - net.want(a)[q]
+        for s in ([200], [70, 1, 1, 40, 2], [1]):
+            base = logits(a, s)[q]
+            assert torch.equal(logits(c, s)[q], base), (q, s)
+            moved = (logits(b, s)[q] - base).double().cpu()
+            assert float((moved - want).norm()) < 0.35 * float(want.norm())
+
+
 @pytest.mark.parametrize("device", DEVICES)
 def test_far_key_among_many(tmp_path, device):
     """One key far back that stands out from hundreds of others, at block and
@@ -869,6 +899,35 @@ def test_graph_replay_matches_eager(tmp_path, dtype, batch):
         assert err(a, b.double().cpu()) < 1e-6
         for s, t in zip(ge.runner.cache.states, ee.runner.cache.states):
             assert torch.equal(s[:batch], t[:batch])
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("batch", [1, 2, 8, 16])
+def test_graph_replay_at_real_sizes(batch):
+    """Skinny, tile and library products of a real layer, replayed with eager
+    steps of another engine in between."""
+    from dataclasses import replace
+
+    from fei_amd.engine.engine import LocalEngine
+    spec = get_spec("bokenex-1b")
+    spec = replace(spec, name="two-layers", vocab_size=4096,
+                   layers=spec.layers[:2])
+    kw = dict(device=torch.device("cuda"), batch_size=batch, max_seq_len=1024,
+              tokenizer=None)
+    ge, ee = LocalEngine(spec, **kw), LocalEngine(spec, use_hip_graph=False,
+                                                  **kw)
+    prompt = toks(300, 4096, 45)
+    for eng in (ge, ee):
+        eng.prefill(prompt)
+    for _ in range(6):
+        ge._graph.replay()
+        torch.cuda.synchronize()
+        ee._decode_step()
+        torch.cuda.synchronize()
+        assert torch.equal(ge.token, ee.token)
+        for a, b in zip(ge.runner.cache.rows, ee.runner.cache.rows):
+            assert torch.equal(a[:64], b[:64])
+    assert err(ge._decode_logits(), ee._decode_logits().double().cpu()) < 1e-6
 
 
 # -- command line -----------------------------------------------------------------------
