@@ -246,24 +246,24 @@ __device__ __forceinline__ int key_place(int key) {
   return (key & 32) + ((key & 15) >> 2) * 8 + ((key >> 4) & 1) * 4 + (key & 3);
 }
 
-// Attention of prompt portions. grid (heads, query tiles, 128 / (16 NW)); a
-// wave owns 16 queries, the block walks the keys they see in tiles of 64 held
-// in LDS: keys row-major, values transposed. The distance bias depends on
-// query - key alone: a tile's NW * 16 + 63 values are computed once, in four
-// copies shifted by one each, so that a lane reads the four of its keys as
-// one aligned vector.
+// Attention of prompt portions. grid (heads, query tiles, 128 / (16 NW QS)); a
+// wave owns QS sets of 16 queries, which share the fragments it reads, the
+// block walks the keys they see in tiles of 64 held in LDS: keys row-major,
+// values transposed. The distance bias depends on query - key alone: a tile's
+// NW * 16 * QS + 63 values are computed once, in four copies shifted by one
+// each, so that a lane reads the four of its keys as one aligned vector.
 // KS >= ceil(dim / 32), DC >= ceil(vdim / 16); queries are zero beyond dim,
 // columns beyond vdim are not stored.
-template <typename T, int KS, int DC, int NW>
+template <typename T, int KS, int DC, int NW, int QS, bool VEC>
 __global__ void __launch_bounds__(NW * 64, 2)
 k_sig_prefill(T* __restrict__ out, long os, const T* __restrict__ q,
               const T* __restrict__ rows, const float* __restrict__ bias,
               const int* __restrict__ spans, const int* __restrict__ tiles,
               const int* __restrict__ table, int seq0, int W, int bs_log,
-              Geo g, int vec) {
+              Geo g) {
   typedef typename El<T>::frag frag;
   constexpr int NP = Parts<T>::n;
-  constexpr int NT = NW * 64, NQ = NW * 16;
+  constexpr int NT = NW * 64, NQ = NW * 16 * QS;
   constexpr int DS = KS * 32 + 8;          // odd count of 16-byte slots
   constexpr int TB = NQ + 68;
   extern __shared__ __align__(16) char smem[];
@@ -272,49 +272,54 @@ k_sig_prefill(T* __restrict__ out, long os, const T* __restrict__ q,
   float* tb = (float*)(vt + DC * 16 * 64);  // [4][TB]
 
   const int h = blockIdx.x, gk = h / (g.heads / g.kvh);
-  const int pt = tiles[blockIdx.y * 2];
+  // a portion's last queries see the most keys: they start first
+  const int tile = gridDim.y - 1 - blockIdx.y;
+  const int pt = tiles[tile * 2];
   const int row0 = spans[pt * 3], cnt = spans[pt * 3 + 1];
   const int pos0 = spans[pt * 3 + 2];
-  const int q0 = tiles[blockIdx.y * 2 + 1] + blockIdx.z * NQ;
+  const int q0 = tiles[tile * 2 + 1] + blockIdx.z * NQ;
   if (q0 >= cnt) return;
   const int qn = min(NQ, cnt - q0);
-  const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63;
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int l15 = lane & 15, lg = lane >> 4;
   const int R = g.kvh * (g.dim + g.vdim);
   const T* kh = rows + (long)gk * g.dim;
   const T* vh = rows + (long)g.kvh * g.dim + (long)gk * g.vdim;
 
-  frag bq[KS];
-  {
-    const int r = min(w * 16 + l15, qn - 1);
+  frag bq[QS][KS];
+  f32x4 o[QS][DC];
+#pragma unroll
+  for (int i = 0; i < QS; ++i) {
+    const int r = min((w * QS + i) * 16 + l15, qn - 1);
     const T* src = q + (long)(row0 - seq0 + q0 + r) * g.heads * g.dim +
                    (long)h * g.dim;
 #pragma unroll
     for (int k = 0; k < KS; ++k) {
       const int c = k * 32 + 8 * lg;
 #pragma unroll
-      for (int j = 0; j < 8; ++j) bq[k][j] = 0;
-      if (vec) {
-        if (c < g.dim) bq[k] = ld8(src + c);
+      for (int j = 0; j < 8; ++j) bq[i][k][j] = 0;
+      if (VEC) {
+        if (c < g.dim) bq[i][k] = ld8(src + c);
       } else {
 #pragma unroll
         for (int j = 0; j < 8; ++j)
-          if (c + j < g.dim) bq[k][j] = src[c + j];
+          if (c + j < g.dim) bq[i][k][j] = src[c + j];
       }
     }
-  }
-  f32x4 o[DC];
 #pragma unroll
-  for (int d = 0; d < DC; ++d) o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int d = 0; d < DC; ++d) o[i][d] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
 
   // positions of this tile's queries and of the keys any of them sees
   const int qa = pos0 + q0, qb = qa + qn - 1;
   const int klo = first_key(qa, g.window) & ~63;
   // this wave's own range: tiles outside it are staged for the others only
-  const int wa = qa + w * 16, wb = min(wa + 15, qb);
+  const int wa = qa + w * 16 * QS, wb = min(wa + 16 * QS - 1, qb);
   const int wlo = first_key(wa, g.window);
   const float r1 = bias[h], r2 = bias[g.heads + h], pb = bias[2 * g.heads + h];
   const float scale = -g.scale * El<T>::base;
+  const unsigned seen = g.window > 0 ? g.window : 1u << 31;
 
   // Cached rows of a tile's keys. Keys past the last query are read as that
   // query's own: their weights are zero, their values have to be finite.
@@ -347,11 +352,11 @@ k_sig_prefill(T* __restrict__ out, long os, const T* __restrict__ q,
       vb[u] = ld8(vh + row_of(first, t0, r + 1) * R + c);
     }
   };
-  if (vec) load(klo);
+  if (VEC) load(klo);
 
   for (int t0 = klo; t0 <= qb; t0 += 64) {
     __syncthreads();
-    if (vec) {
+    if (VEC) {
 #pragma unroll
       for (int u = 0; u < UK; ++u) {
         const int i = tid + u * NT;
@@ -391,67 +396,87 @@ k_sig_prefill(T* __restrict__ out, long os, const T* __restrict__ q,
         if (i >= s) tb[s * TB + i - s] = v;
     }
     __syncthreads();
-    if (vec && t0 + 64 <= qb) load(t0 + 64);
+    if (VEC && t0 + 64 <= qb) load(t0 + 64);
     if (t0 > wb || t0 + 63 < wlo) continue;
 
-    f32x4 s[4];
+    f32x4 s[QS][4];
 #pragma unroll
     for (int c = 0; c < 4; ++c) {
-      s[c] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int k = 0; k < KS; ++k)
-        s[c] = mma(ld8(kt + (c * 16 + l15) * DS + k * 32 + 8 * lg), bq[k],
-                   s[c]);
+      for (int i = 0; i < QS; ++i) s[i][c] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int k = 0; k < KS; ++k) {
+        const frag a = ld8(kt + (c * 16 + l15) * DS + k * 32 + 8 * lg);
+#pragma unroll
+        for (int i = 0; i < QS; ++i) s[i][c] = mma(a, bq[i][k], s[i][c]);
+      }
     }
     // no mask where every query of the wave sees every key of the tile
     const bool edge = t0 + 63 > wa || (g.window > 0 && wb - t0 >= g.window);
-    const int qp = wa + l15, sh = (3 - l15) & 3;
-    const float* tq = tb + sh * TB + 4 * lg - w * 16 - l15 + NQ - 1 - sh;
+    const int sh = (3 - l15) & 3;
 #pragma unroll
-    for (int c = 0; c < 4; ++c) {
-      const f32x4 b = *(const f32x4*)(tq + c * 16);
+    for (int i = 0; i < QS; ++i) {
+      const int qp = wa + i * 16 + l15;
+      const float* tq = tb + sh * TB + 4 * lg - (w * QS + i) * 16 - l15 + NQ -
+                        1 - sh;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        float v = El<T>::inv(1.f + El<T>::exb(fmaf(s[c][r], scale, b[r])));
-        if (edge) {
-          const int d = qp - (t0 + c * 16 + 4 * lg + r);
-          if (d < 0 || (g.window > 0 && d >= g.window)) v = 0.f;
-        }
-        s[c][r] = v;
+      for (int c = 0; c < 4; ++c) {
+        const f32x4 b = *(const f32x4*)(tq + c * 16);
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          s[i][c][r] =
+              El<T>::inv(1.f + El<T>::exb(fmaf(s[i][c][r], scale, b[r])));
+      }
+      if (edge) {
+        const int d0 = qp - t0 - 4 * lg;
+#pragma unroll
+        for (int c = 0; c < 4; ++c)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const unsigned d = d0 - c * 16 - r;   // a key ahead: huge
+            if (d >= seen) s[i][c][r] = 0.f;
+          }
       }
     }
 #pragma unroll
     for (int k = 0; k < 2; ++k) {
-      frag pw[NP];
+      frag pw[QS][NP];
 #pragma unroll
-      for (int j = 0; j < 8; ++j)
+      for (int i = 0; i < QS; ++i) {
+        float v[8];
 #pragma unroll
-        for (int i = 0; i < NP; ++i)
-          pw[i][j] = part_of<T>(s[2 * k + (j >> 2)][j & 3], i);
+        for (int j = 0; j < 8; ++j) v[j] = s[i][2 * k + (j >> 2)][j & 3];
+        weight_parts(v, pw[i]);
+      }
 #pragma unroll
       for (int d = 0; d < DC; ++d) {
         const frag av = ld8(vt + vt_at(d * 16 + l15, k * 32 + 8 * lg));
 #pragma unroll
-        for (int i = 0; i < NP; ++i) o[d] = mma(av, pw[i], o[d]);
+        for (int i = 0; i < QS; ++i)
+#pragma unroll
+          for (int n = 0; n < NP; ++n) o[i][d] = mma(av, pw[i][n], o[i][d]);
       }
     }
   }
 
-  const int r = w * 16 + l15;
-  if (r >= qn) return;
-  T* dst = out + (long)(row0 + q0 + r) * os + (long)h * g.vdim;
 #pragma unroll
-  for (int d = 0; d < DC; ++d) {
-    const int c = d * 16 + 4 * lg;
-    T v[4];
+  for (int i = 0; i < QS; ++i) {
+    const int r = (w * QS + i) * 16 + l15;
+    if (r >= qn) continue;
+    T* dst = out + (long)(row0 + q0 + r) * os + (long)h * g.vdim;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) v[i] = El<T>::st(o[d][i]);
-    if (vec) {
-      if (c < g.vdim) __builtin_memcpy(dst + c, v, sizeof(v));
-    } else {
+    for (int d = 0; d < DC; ++d) {
+      const int c = d * 16 + 4 * lg;
+      T v[4];
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
-        if (c + i < g.vdim) dst[c + i] = v[i];
+      for (int j = 0; j < 4; ++j) v[j] = El<T>::st(o[i][d][j]);
+      if (VEC) {
+        if (c < g.vdim) __builtin_memcpy(dst + c, v, sizeof(v));
+      } else {
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          if (c + j < g.vdim) dst[c + j] = v[j];
+      }
     }
   }
 }
@@ -493,7 +518,8 @@ k_sig_decode(T* __restrict__ out, long os, float* __restrict__ part,
   const int hg = g.heads / g.kvh, ht = (hg + 15) / 16;
   const int gk = blockIdx.y / ht, hy = blockIdx.y - gk * ht;
   const int h0 = gk * hg + hy * 16, nh = min(16, hg - hy * 16);
-  const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63;
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int l15 = lane & 15, lg = lane >> 4;
   const int R = g.kvh * (g.dim + g.vdim), CH = channels(g);
   const int p = pos[b], k0 = first_key(p, g.window);
@@ -664,6 +690,7 @@ k_sig_decode(T* __restrict__ out, long os, float* __restrict__ part,
         }
     }
     frag pw[NP];
+    float pv[8];
 #pragma unroll
     for (int c = 0; c < 2; ++c) {
       f32x4 s = {0.f, 0.f, 0.f, 0.f};
@@ -676,10 +703,10 @@ k_sig_decode(T* __restrict__ out, long os, float* __restrict__ part,
         const float off = (r1 * El<T>::ln(1.f + r2 * d) - pb) * El<T>::base;
         float v = El<T>::inv(1.f + El<T>::exb(fmaf(s[r], scale, off)));
         if (key > p || key < k0) v = 0.f;
-#pragma unroll
-        for (int i = 0; i < NP; ++i) pw[i][c * 4 + r] = part_of<T>(v, i);
+        pv[c * 4 + r] = v;
       }
     }
+    weight_parts(pv, pw);
 #pragma unroll
     for (int i = 0; i < CPL; ++i) {
       frag av;
@@ -826,23 +853,26 @@ void run_conv(T* q, const T* proj, long ps, T* rows, float* states, Conv cv,
                        cv.taps, CH);
 }
 
-template <typename T, int KS, int DC>
+template <typename T, int KS, int DC, bool VEC>
 void launch_prefill(T* out, long os, const T* q, const T* rows,
                     const float* bias, const int* spans, const int* tiles,
                     const int* table, int n_tiles, int seq0, int W, int bs_log,
-                    Geo g, int vec, hipStream_t stream) {
-  constexpr int NW = sizeof(T) == 2 ? 8 : 4;
+                    Geo g, hipStream_t stream) {
+  // the registers of two sets of queries suffice up to these sizes
+  constexpr int QS = sizeof(T) == 2 && KS <= 4 && DC <= 8 ? 2 : 1;
+  constexpr int NW = sizeof(T) == 2 ? 8 / QS : 4;
+  constexpr int NQ = NW * 16 * QS;
   static bool set = false;
   if (!set) {
-    allow_lds(k_sig_prefill<T, KS, DC, NW>);
+    allow_lds(k_sig_prefill<T, KS, DC, NW, QS, VEC>);
     set = true;
   }
   const size_t lds = sizeof(T) * (64 * (KS * 32 + 8) + DC * 16 * 64) +
-                     16 * (NW * 16 + 68);
-  const dim3 grid(g.heads, n_tiles, NW == 8 ? 1 : 2);
-  hipLaunchKernelGGL((k_sig_prefill<T, KS, DC, NW>), grid, dim3(NW * 64), lds,
-                     stream, out, os, q, rows, bias, spans, tiles, table, seq0,
-                     W, bs_log, g, vec);
+                     16 * (NQ + 68);
+  const dim3 grid(g.heads, n_tiles, 128 / NQ);
+  hipLaunchKernelGGL((k_sig_prefill<T, KS, DC, NW, QS, VEC>), grid,
+                     dim3(NW * 64), lds, stream, out, os, q, rows, bias,
+                     spans, tiles, table, seq0, W, bs_log, g);
 }
 
 template <typename T>
@@ -850,17 +880,17 @@ void run_prefill(T* out, long os, const T* q, const T* rows,
                  const float* bias, const int* spans, const int* tiles,
                  const int* table, int n_tiles, int seq0, int W, int bs_log,
                  Geo g, hipStream_t stream) {
-  const int vec = g.dim % 8 == 0 && g.vdim % 8 == 0 && os % 4 == 0;
-#define PRE(KS, DC) launch_prefill<T, KS, DC>(out, os, q, rows, bias, spans, \
-                                              tiles, table, n_tiles, seq0, W, \
-                                              bs_log, g, vec, stream)
-#define BY_DC(KS)                       \
-  do {                                  \
-    if (g.vdim <= 64) PRE(KS, 4);       \
-    else if (g.vdim <= 128) PRE(KS, 8); \
-    else PRE(KS, 16);                   \
+#define PRE(KS, DC, VEC)                                                     \
+  launch_prefill<T, KS, DC, VEC>(out, os, q, rows, bias, spans, tiles,       \
+                                 table, n_tiles, seq0, W, bs_log, g, stream)
+#define BY_DC(KS)                             \
+  do {                                        \
+    if (g.vdim <= 64) PRE(KS, 4, true);       \
+    else if (g.vdim <= 128) PRE(KS, 8, true); \
+    else PRE(KS, 16, true);                   \
   } while (0)
-  if (g.dim <= 64) BY_DC(2);
+  if (g.dim % 8 || g.vdim % 8 || os % 4) PRE(8, 16, false);
+  else if (g.dim <= 64) BY_DC(2);
   else if (g.dim <= 128) BY_DC(4);
   else BY_DC(8);
 #undef BY_DC
