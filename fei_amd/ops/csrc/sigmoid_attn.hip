@@ -497,7 +497,8 @@ __device__ __forceinline__ void split_of(int p, int window, int splits,
 // and reads them from LDS. Split 0 writes the state.
 // A lane holds CPL value columns: CPL * 16 >= vdim. KS >= ceil(dim / 32).
 template <typename T, int KS, int CPL, bool VEC>
-__global__ void __launch_bounds__(256)
+__global__ void
+__launch_bounds__(256, sizeof(T) == 2 && KS <= 4 && CPL <= 8 ? 2 : 1)
 k_sig_decode(T* __restrict__ out, long os, float* __restrict__ part,
              const T* __restrict__ proj, long ps, T* __restrict__ rows,
              float* __restrict__ states, Conv cv,
@@ -518,8 +519,7 @@ k_sig_decode(T* __restrict__ out, long os, float* __restrict__ part,
   const int hg = g.heads / g.kvh, ht = (hg + 15) / 16;
   const int gk = blockIdx.y / ht, hy = blockIdx.y - gk * ht;
   const int h0 = gk * hg + hy * 16, nh = min(16, hg - hy * 16);
-  const int tid = threadIdx.x, lane = tid & 63;
-  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63;
   const int l15 = lane & 15, lg = lane >> 4;
   const int R = g.kvh * (g.dim + g.vdim), CH = channels(g);
   const int p = pos[b], k0 = first_key(p, g.window);
