@@ -190,80 +190,131 @@ k_moe_gemm(T* __restrict__ out, const T* __restrict__ x,
   }
 }
 
-// 64 lanes x 16 bytes from memory straight into LDS, lane i at lds + 16 i.
-__device__ __forceinline__ void load_lds(const u16* src, u16* lds) {
-  __builtin_amdgcn_global_load_lds(
-      (const __attribute__((address_space(1))) void*)src,
-      (__attribute__((address_space(3))) void*)lds, 16, 0, 0);
+// 64 lanes x 16 bytes from memory straight into LDS, lane i at lds + 16 i
+// (a byte address, the same in all lanes).
+__device__ __forceinline__ void load_lds(const u16* src, u32 lds) {
+  u32 keep;
+  asm volatile(
+      "s_mov_b32 %0, m0\n\t"
+      "s_mov_b32 m0, %2\n\t"
+      "s_nop 0\n\t"
+      "global_load_lds_dwordx4 %1, off\n\t"
+      "s_mov_b32 m0, %0"
+      : "=&s"(keep)
+      : "v"(src), "s"(lds)
+      : "memory");
 }
 
 // The same for bfloat16 with K % 64 == 0 and N % 4 == 0: tiles of 128 slots x
-// 128 columns, 4 waves of 64 x 64, two LDS buffers of 64 steps of K filled by
-// direct loads. The 16-byte places of a row are permuted by the row (in the
-// address that a lane reads, since LDS is filled in lane order), so that the
-// fragment reads of 16 rows spread over the banks.
+// 32 WI columns, 4 waves of 64 slots x 16 WI columns, S LDS buffers of 64
+// steps of K filled by direct loads. The 16-byte places of a row are permuted
+// by the row (in the address that a lane reads, since LDS is filled in lane
+// order), so that the fragment reads of 16 rows spread over the banks.
+// An XCD gets consecutive blocks, in groups of 8 tiles of slots times all nx of
+// columns, slots first: its L2 then holds their common rows and weights.
+template <int WI, int S>
 __global__ void __launch_bounds__(256, 2)
 k_moe_gemm_big(u16* __restrict__ out, const u16* __restrict__ x,
                const u16* __restrict__ w, const int* __restrict__ order,
                const int* __restrict__ tiles, const int* __restrict__ count,
-               int N, int K, int act) {
-  __shared__ __align__(16) u16 buf[2][2][128 * 64];
-  if ((int)blockIdx.y >= count[0]) return;
-  const int* t = tiles + blockIdx.y * 3;
-  const int s0 = t[1], cnt = t[2], n0 = blockIdx.x * 128;
+               int nx, int N, int K, int act) {
+  constexpr int TN = 32 * WI;
+  constexpr int BUF = (128 + TN) * 64;     // elements: 128 rows of x, TN of w
+  constexpr int LOADS = 4 + WI;            // a wave's per buffer: x, w
+  extern __shared__ __align__(16) u16 buf[];
+  const int total = count[0] * nx, per = (total + 7) / 8;
+  const int id = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+  if ((int)(blockIdx.x >> 3) >= per || id >= total) return;
+  const int g0 = id / (8 * nx) * 8, gm = min(8, count[0] - g0);
+  const int gr = id - g0 * nx;
+  const int* t = tiles + (g0 + gr % gm) * 3;
+  const int s0 = t[1], cnt = t[2], n0 = gr / gm * TN;
   const u16* we = w + (long)t[0] * N * K;
-  const int tid = threadIdx.x, wid = tid >> 6, lane = tid & 63;
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int l15 = lane & 15, lg = lane >> 4;
-  const u16* src[2][4];
+  // 8 rows a load; the place of a row's 8 values depends on the row
+  const int r8 = lane >> 3, c8 = ((lane & 7) ^ r8) * 8;
+  const u16* src[LOADS];
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
-    const int r = (wid * 4 + i) * 8 + (lane >> 3);
-    const int c = ((lane & 7) ^ (r & 7)) * 8;
-    const int slot = s0 + min(r, cnt - 1);
-    src[0][i] = x + (long)(order ? order[slot] : slot) * K + c;
-    src[1][i] = we + (long)min(n0 + r, N - 1) * K + c;
+    const int slot = s0 + min((wid * 4 + i) * 8 + r8, cnt - 1);
+    src[i] = x + (long)(order ? order[slot] : slot) * K + c8;
   }
-  auto stage = [&](int b, int k0) {
 #pragma unroll
-    for (int m = 0; m < 2; ++m)
-#pragma unroll
-      for (int i = 0; i < 4; ++i)
-        load_lds(src[m][i] + k0, &buf[b][m][(wid * 4 + i) * 512]);
+  for (int i = 0; i < WI; ++i)
+    src[4 + i] = we + (long)min(n0 + (wid * WI + i) * 8 + r8, N - 1) * K + c8;
+  const u32 lds = (u32)(uintptr_t)(__attribute__((address_space(3))) u16*)buf;
+  const int steps = K / 64;
+  // past the end the last steps are read again, into a buffer that is free
+  auto load = [&](int step, int b, int i) {
+    load_lds(src[i] + min(step, steps - 1) * 64,
+             lds + b * BUF * 2 +
+                 (i < 4 ? (wid * 4 + i) * 1024
+                        : 16384 + (wid * WI + i - 4) * 1024));
   };
-  const int xm = (wid & 1) * 64, wm = (wid >> 1) * 64;
-  f32x4 acc[4][4];
+  const int xm = (wid & 1) * 64, wm = (wid >> 1) * 16 * WI;
+  struct Frags {
+    s16x8 w[WI], x[4];
+  };
+  auto read = [&](Frags& f, int b, int kk, int i) {
+    const int c = ((kk * 4 + lg) ^ (l15 & 7)) * 8;
+    const u16* bx = buf + b * BUF;
+    if (i < 4) f.x[i] = ld8(bx + (xm + i * 16 + l15) * 64 + c);
+    f.w[i] = ld8(bx + (128 + wm + i * 16 + l15) * 64 + c);
+  };
+  f32x4 acc[WI][4];
 #pragma unroll
-  for (int i = 0; i < 4; ++i)
+  for (int i = 0; i < WI; ++i)
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  stage(0, 0);
-  int b = 0;
-  for (int k0 = 0; k0 < K; k0 += 64, b ^= 1) {
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    __syncthreads();         // this buffer is full, the other one read
-    if (k0 + 64 < K) stage(b ^ 1, k0 + 64);
 #pragma unroll
-    for (int k = 0; k < 2; ++k) {
-      s16x8 fa[4], fx[4];
-      const int c = ((k * 4 + lg) ^ (l15 & 7)) * 8;
+  for (int s = 0; s < S; ++s)
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        fa[i] = ld8(&buf[b][1][(wm + i * 16 + l15) * 64 + c]);
-        fx[i] = ld8(&buf[b][0][(xm + i * 16 + l15) * 64 + c]);
-      }
+    for (int i = 0; i < LOADS; ++i) load(s, s, i);
+  asm volatile("s_waitcnt vmcnt(%0)\n\ts_barrier" ::"n"((S - 1) * LOADS)
+               : "memory");
+  Frags f0, f1;
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
+  for (int i = 0; i < WI; ++i) read(f0, 0, 0, i);
+  int b = 0;                               // buffer of step k
+  // Fragments of 32 steps of K are read ahead of the products with the 32
+  // before. At the barrier all waves have the second half of buffer b, which
+  // can be filled again, and the loads of the next one have arrived. Reads
+  // and loads go out between the matrix instructions.
+  for (int k = 0; k < steps; ++k) {
 #pragma unroll
-        for (int j = 0; j < 4; ++j) acc[i][j] = mma(fa[i], fx[j], acc[i][j]);
+    for (int i = 0; i < WI; ++i) {
+      read(f1, b, 1, i);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        acc[i][j] = mma(f0.w[i], f0.x[j], acc[i][j]);
+      __builtin_amdgcn_sched_barrier(0);
     }
+    asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"(
+                     (S - 2) * LOADS)
+                 : "memory");
+    const int nb = b == S - 1 ? 0 : b + 1;
+#pragma unroll
+    for (int i = 0; i < WI; ++i) {
+      read(f0, nb, 0, i);
+      load(k + S, b, i);
+      if (WI + i < LOADS) load(k + S, b, WI + i);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        acc[i][j] = mma(f1.w[i], f1.x[j], acc[i][j]);
+      __builtin_amdgcn_sched_barrier(0);
+    }
+    b = nb;
   }
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
     const int r = xm + j * 16 + l15;
     if (r >= cnt) continue;
     u16* dst = out + (long)(s0 + r) * N;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
+    for (int i = 0; i < WI; ++i) {
       const int n = n0 + wm + i * 16 + 4 * lg;
       if (n >= N) continue;
       u16 v[4];
@@ -273,6 +324,24 @@ k_moe_gemm_big(u16* __restrict__ out, const u16* __restrict__ x,
       __builtin_memcpy(dst + n, v, sizeof(v));
     }
   }
+}
+
+template <int WI, int S>
+void launch_big(u16* out, const u16* x, const u16* w, const int* order,
+                const int* tiles, const int* count, int max_tiles, int N,
+                int K, int act, hipStream_t stream) {
+  constexpr int lds = S * (128 + 32 * WI) * 64 * 2;
+  static bool set = false;
+  if (!set) {
+    (void)hipFuncSetAttribute((const void*)k_moe_gemm_big<WI, S>,
+                              hipFuncAttributeMaxDynamicSharedMemorySize,
+                              lds);
+    set = true;
+  }
+  const int nx = (N + 32 * WI - 1) / (32 * WI);
+  hipLaunchKernelGGL((k_moe_gemm_big<WI, S>),
+                     dim3((nx * max_tiles + 7) / 8 * 8), dim3(256), lds,
+                     stream, out, x, w, order, tiles, count, nx, N, K, act);
 }
 
 // x[t] += mult * sum_k w[t, k] y[place[t, k]]. One block per row.
@@ -457,9 +526,14 @@ void fei_moe_gemm(void* out, const void* x, const void* w, const int* order,
                   const int* tiles, const int* count, int max_tiles, int N,
                   int K, int act, int bits, hipStream_t stream) {
   if (bits & 2) {
-    hipLaunchKernelGGL(k_moe_gemm_big, dim3((N + 127) / 128, max_tiles),
-                       dim3(256), 0, stream, (u16*)out, (const u16*)x,
-                       (const u16*)w, order, tiles, count, N, K, act);
+    // 192 columns a block unless they are wasted or leave CUs without a block
+    const int c6 = (N + 191) / 192, c4 = (N + 127) / 128;
+    if (c6 * max_tiles >= 512 && c6 * 192 * 10 <= c4 * 128 * 11)
+      launch_big<6, 2>((u16*)out, (const u16*)x, (const u16*)w, order, tiles,
+                       count, max_tiles, N, K, act, stream);
+    else
+      launch_big<4, 2>((u16*)out, (const u16*)x, (const u16*)w, order, tiles,
+                       count, max_tiles, N, K, act, stream);
     return;
   }
   const dim3 grid((N + 63) / 64, max_tiles);

@@ -229,7 +229,7 @@ def experts_want(x, gain, eps, a, w_o, up, down, router, f, mult):
 # experts, top, their width, width: scalar sizes, sizes of the skinny and of
 # the tiled products, more experts than rows
 MOE_SIZES = [(5, 2, 21, 52), (6, 3, 64, 128), (4, 2, 192, 1024),
-             (40, 4, 72, 64), (3, 1, 128, 320)]
+             (40, 4, 72, 64), (3, 1, 128, 320), (2, 2, 640, 192)]
 
 
 MOE_CASES = [("cpu", torch.float32, n) for n in (1, 9)] + [
@@ -276,6 +276,34 @@ def test_experts(device, dtype, rows, size):
                         d(router), f, mult)
     assert err(got - x.to(device), want - d(x)) < (
         2e-5 if dtype == torch.float32 else 1.2e-2)
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("size", [(8, 2, 1536, 1536), (3, 2, 64, 3072)])
+def test_many_experts_rows(size):
+    """Enough tiles for the widest blocks of the grouped product, the last of
+    each expert not full."""
+    E, top, ff, C = size
+    T = 4001
+    g = torch.Generator(device="cuda").manual_seed(T)
+    rand = lambda *s: torch.randn(*s, generator=g, device="cuda")
+    x = rand(T, C)
+    up, down = ((rand(E, *s) / s[1] ** 0.5).bfloat16()
+                for s in ((ff, C), (C, ff)))
+    z = rand(T, E) * 3.0
+    w_o, a = torch.zeros(C, 8, device="cuda").bfloat16(), \
+        torch.zeros(T, 8, device="cuda").bfloat16()
+    norm = ops.GainNorm(torch.ones((), device="cuda"), C, 1e-5)
+    h = ops.GainNormed(x, norm, torch.bfloat16)
+    rows = h.rows.clone()
+    f = MoESpec(E, top, ff, 1.0)
+    got = ops.residual_moe(torch.zeros_like(x), h, z, a, w_o, up, down, f, 1.0)
+    ids, w = ops.ref.route(z.cpu(), top, 1.0)
+    some = torch.randperm(T, generator=torch.Generator().manual_seed(1))[:64]
+    want = ops.ref.moe(rows[some].float().cpu(), ids[some], w[some],
+                       up.float().cpu(), down.float().cpu())
+    assert err(got[some], want) < 1.2e-2
+    assert bool(torch.isfinite(got).all())
 
 
 @pytest.mark.gpu
