@@ -332,7 +332,7 @@ class PagedSessionManager:
 
 
 class StepSessionManager(PagedSessionManager):
-    """Sessions over a StepRunner: one cache of latent rows and state slots,
+    """Sessions over a StepRunner: one cache of rows and state slots,
     one ragged batch per step.
 
     ``open`` admits a session (a state slot, and blocks for its prompt) and
